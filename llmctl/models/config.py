@@ -298,6 +298,12 @@ def get_model_config(name_or_path: str) -> ModelConfig:
         kv = {p[0]: int(p[1:]) for p in key.split("-")[1:] if p[1:].isdigit()}
         return pamazen_template(width=kv.get("w", 256), layers=kv.get("l", 4), heads=kv.get("h", 4),
                                 kv_heads=kv.get("g", 2), experts=kv.get("e", 8), streams=kv.get("s", 4))
+    if key.startswith("dapipel-"):  # dapipel-w<width>-l<layers>[-h<heads>][-g<kv heads>][-e<experts>]: random-init template
+        from .dapipel import dapipel_template
+
+        kv = {p[0]: int(p[1:]) for p in key.split("-")[1:] if p[1:].isdigit()}
+        return dapipel_template(width=kv.get("w", 256), layers=kv.get("l", 4), heads=kv.get("h", 4),
+                                kv_heads=kv.get("g", 2), experts=kv.get("e", 0))
     if key in ALIASES:
         t, s = ALIASES[key]
         return ModelConfig.from_dict(MODEL_TEMPLATES[t][s])

@@ -21,7 +21,12 @@
   cache ``[v | k]``: biases on q / k / v, RMS norm over the whole of q and of k, a query temperature that
   grows with the logarithm of the position, a logarithmic distance penalty per head, key weights
   ``sigmoid(score + head bias)`` that are not normalised, one sigmoid output gate per head.
-* :class:`DenseFF` — an ungated feed-forward ``W_down act(W_up h)``.
+* :class:`DenseFF` — an ungated feed-forward ``W_down act(W_up h)``; :class:`GatedFF` — a gated one, ``W_down
+  (act(W_gate h) * W_up h)``.
+* :class:`DifferentialAttention` — grouped-query attention with two softmax maps per head over the same values whose
+  outputs are subtracted (a learned factor), RMS-normed per head and scaled; paged rows ``[v | k_1 | k_2]``.
+* :class:`MinGRU` — an elementwise gated recurrence whose gates read only the current token, with an output gate;
+  one fp32 vector per state slot.
 * :class:`DeltaRule` — the generalized delta rule: a matrix memory per head that decays per key channel, removes
   what it holds along the current unit key at a learned rate and then writes ``k v^T``; low-rank decay projection
   through a ``tanh``, per-head unit RMS, weight and sigmoid gate on the read-out; state in a slot pool.
@@ -73,6 +78,7 @@ class StepBatch:
     cu_host: Optional[list] = None  # ``cu`` on the host (chunk-parallel scans split long portions)
     seq_of: Optional[torch.Tensor] = None  # int32 [T] index (into cu / start / state) of every row's sequence
     d_max_ctx: int = 0  # the longest context among the decoding sequences
+    carried: bool = True  # some prompt portion of more than one row continues a sequence (its first position is not 0)
     fresh: bool = False  # every row belongs to a prompt portion that starts at position 0 (no earlier context)
     scratch: dict = field(default_factory=dict)  # what layers derive from the step alone and share (chunk plans of scans)
 
@@ -164,6 +170,13 @@ class LatentAttention(nn.Module):
             self._uvk_key = key
         return self._uvk
 
+    def _w_uv_t(self) -> torch.Tensor:
+        """W_uv per head as ``[H, rank, vdim]`` rows (made once): the right operand of a batched product is contiguous."""
+        key = (self.w_uv.data_ptr(), self.w_uv._version)
+        if getattr(self, "_uvt_key", None) != key:
+            self._uvt, self._uvt_key = self.w_uv.detach().transpose(1, 2).contiguous(), key
+        return self._uvt
+
     def _attend_expanded(self, q: torch.Tensor, b: StepBatch, cache: torch.Tensor) -> torch.Tensor:
         T, H, dn, dr, dv = q.shape[0], self.H, self.dn, self.dr, self.dv
         lat = cache.view(-1, self.rk + dr).index_select(0, b.slots)  # the rows just written: [latent | rotary key]
@@ -205,7 +218,7 @@ class LatentAttention(nn.Module):
             outs.append(hops.latent_attention_decode(qa[b.Tp:], cache, b.d_bt, b.d_ctx, self.window, self.sink,
                                                      self.scale, self.rk, max_ctx=b.d_max_ctx))
         o_lat = outs[0] if len(outs) == 1 else torch.cat(outs)
-        o = torch.bmm(o_lat.transpose(0, 1), self.w_uv.transpose(1, 2)).transpose(0, 1).reshape(T, H * self.dv)
+        o = torch.bmm(o_lat.transpose(0, 1), self._w_uv_t()).transpose(0, 1).reshape(T, H * self.dv)
         if self.has_gate:
             o = hops.sigmoid_gate_mul(o, z[:, c:])
         return F.linear(o, self.w_o)
@@ -539,6 +552,113 @@ class DenseFF(nn.Module):
         z = F.linear(h, self.w_up, self.b_up)
         y = F.linear(hops.act_any(z[:, :self.ff], self.act), self.w_down)
         return (y, z[:, self.ff:]) if self.side else y
+
+
+class GatedFF(nn.Module):
+    """``W_down (act(W_gate h) * W_up h)`` with ``act`` one of :func:`llmctl.ops.hybrid.glu_act`'s kinds; gate and up
+    are one weight ``[gate ; up]``."""
+
+    def __init__(self, width: int, ff: int, act: str = "silu", device=None, dtype=None):
+        super().__init__()
+        self.ff, self.act = ff, act
+        self.w_gu = nn.Parameter(torch.empty(2 * ff, width, device=device, dtype=dtype))
+        self.w_down = nn.Parameter(torch.empty(width, ff, device=device, dtype=dtype))
+        _init(self.w_gu, 0.02)
+        _init(self.w_down, 0.02)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return F.linear(hops.glu_act(F.linear(h, self.w_gu), self.act), self.w_down)
+
+
+class DifferentialAttention(nn.Module):
+    """Grouped-query attention with two maps per head (``heads`` query heads over ``kv_heads`` key / value heads; key size
+    ``dim`` per map, value size ``vdim``): both maps are ordinary softmax attentions of their own queries and keys over
+    the same values, no rotation, scores times ``scale``, inside a causal ``window``.  With the maps' outputs
+    ``a_1, a_2`` and ``lam = exp(sum lq1 lk1) - exp(sum lq2 lk2) + diff`` (one number for all heads) a head gives
+    ``o = a_1 - lam a_2``, then ``(1 - diff) o / rms(o)``.  The fused weight is ``[W_q ; W_k ; W_v]`` with ``W_q`` and
+    ``W_k`` head by head as ``[map 1 ; map 2]``; the cache row of a token is ``[v | k_1 | k_2]`` per kv head."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, diff: float, eps: float,
+                 window: Optional[int] = None, device=None, dtype=None):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("kv heads must divide the heads")
+        self.width, self.H, self.G, self.dk, self.dv = width, heads, kv_heads, dim, vdim
+        self.scale, self.diff, self.eps = float(scale), float(diff), eps
+        self.window = int(window) if window else hops.NO_LIMIT
+        kw = dict(device=device, dtype=dtype)
+        self.w_qkv = nn.Parameter(torch.empty(2 * (heads + kv_heads) * dim + kv_heads * vdim, width, **kw))
+        self.w_o = nn.Parameter(torch.empty(width, heads * vdim, **kw))
+        for n in ("lq1", "lk1", "lq2", "lk2"):
+            setattr(self, n, nn.Parameter(torch.zeros(dim, device=device, dtype=torch.float32)))
+        for w in (self.w_qkv, self.w_o):
+            _init(w, 0.02)
+        self._lam, self._lam_key = None, None
+
+    cache_kind = "latent"  # a paged pool of rows
+
+    @property
+    def cache_row(self) -> int:
+        return self.G * (self.dv + 2 * self.dk)
+
+    def state_shapes(self):
+        return []
+
+    def lam(self) -> torch.Tensor:
+        """The factor on the second map, fp32 ``[1]`` (made once; serving weights are static)."""
+        ts = (self.lq1, self.lk1, self.lq2, self.lk2)
+        key = tuple((t.data_ptr(), t._version) for t in ts)
+        if self._lam_key != key:
+            a, b, c, d = (t.detach().float() for t in ts)
+            self._lam = (torch.exp((a * b).sum()) - torch.exp((c * d).sum()) + self.diff).reshape(1)
+            self._lam_key = key
+        return self._lam
+
+    def step(self, h: torch.Tensor, b: StepBatch, cache) -> torch.Tensor:
+        rows = cache[0] if isinstance(cache, tuple) else cache
+        T, H, G, dk, dv = h.shape[0], self.H, self.G, self.dk, self.dv
+        z = F.linear(h, self.w_qkv)
+        k0, v0 = 2 * H * dk, 2 * (H + G) * dk
+        hops.kv_rows_write(z[:, k0:v0], z[:, v0:], rows, b.slots, G)
+        o = torch.empty(T, H * dv, device=h.device, dtype=h.dtype)
+        a = (H, G, dk, dv, self.window, self.scale, self.lam(), 1.0 - self.diff, self.eps)
+        if b.Tp:
+            hops.diff_attention(z[:b.Tp, :k0], rows, b.p_bt, b.p_cu, b.p_ctx, *a, out=o[:b.Tp], max_q=b.max_q)
+        if T > b.Tp:
+            hops.diff_attention(z[b.Tp:, :k0], rows, b.d_bt, None, b.d_ctx, *a, out=o[b.Tp:], max_ctx=b.d_max_ctx)
+        return F.linear(o, self.w_o)
+
+
+class MinGRU(nn.Module):
+    """A gated recurrence whose gates read only the current token, channel by channel over ``state_width`` channels:
+    ``zeta = sigmoid(W_z h + b_z)``, ``u = W_x h + b_x``, candidate ``u + 1/2`` where ``u >= 0`` and ``sigmoid(u)`` elsewhere,
+    ``S_t = (1 - zeta) S_(t-1) + zeta cand``; the result is ``W_o (S_t * silu(W_g h))``.  The state is fp32 and lives in
+    a slot per sequence.  The fused input weight is ``[W_z ; W_x ; W_g]``; the biases stay fp32 and are added inside the
+    scan."""
+
+    def __init__(self, width: int, state_width: int, device=None, dtype=None):
+        super().__init__()
+        self.width, self.n = width, state_width
+        kw = dict(device=device, dtype=dtype)
+        f32 = dict(device=device, dtype=torch.float32)
+        self.w_in = nn.Parameter(torch.empty(3 * state_width, width, **kw))
+        self.b_z = nn.Parameter(torch.zeros(state_width, **f32))
+        self.b_x = nn.Parameter(torch.zeros(state_width, **f32))
+        self.w_o = nn.Parameter(torch.empty(width, state_width, **kw))
+        for w in (self.w_in, self.w_o):
+            _init(w, 0.02)
+
+    cache_kind = "state"
+    cache_row = 0
+
+    def state_shapes(self):
+        return [(self.n,)]
+
+    def step(self, h: torch.Tensor, b: StepBatch, state) -> torch.Tensor:
+        if isinstance(state, tuple) and len(state) == 2 and isinstance(state[1], tuple):  # (rows, states)
+            state = state[1]
+        y = hops.mingru_scan(F.linear(h, self.w_in), self.b_z, self.b_x, state[0], b)
+        return F.linear(y, self.w_o)
 
 
 class DeltaRule(nn.Module):

@@ -234,19 +234,20 @@ class GroupLimitedMoE(nn.Module):
 class BiasedSoftmaxMoE(nn.Module):
     """Routed experts chosen by softmax scores plus a selection bias (serving forward).  Router logits are an
     fp32 product; ``s = softmax(z)``; the ``top`` experts with the largest ``s + bias`` are used, weighted by their
-    own ``s`` (over the sum of the chosen ones when ``renorm``); an optional shared expert of the same form runs
+    own ``s`` (over the sum of the chosen ones when ``renorm``: the softmax over the chosen logits); an optional shared expert of the same form runs
     for every token.  Experts: ``W_down act(W_up h)`` with ``act`` = ``relu2`` / ``gelu``, or gated, ``W_down
     (silu(W_gate h) * W_up h)``, with ``act="swiglu"`` (gate and up are one weight ``[gate ; up]``).  Options:
     ``groups`` / ``keep``: the router's outputs form equal groups of neighbours, a group scores as its best choice
     score, and only experts of the ``keep`` best groups can be chosen; ``identity``: the last that many router
     outputs are experts without weights whose output is their input; ``shared_gate``: the shared expert's output is
-    multiplied by ``sigmoid(w_sg . h)``, one number per token, whose row rides on the shared up projection.
+    multiplied by ``sigmoid(w_sg . h)``, one number per token, whose row rides on the shared up projection;
+    ``select_bias=False``: there is no selection bias.  The experts' down weights are one matrix ``[width, experts * ff]``.
     Dispatch as in :class:`GroupLimitedMoE`
     (token copies sorted by expert, per-expert GEMMs on contiguous segments, fp32 weighted sum).  Steps of
     few tokens that between them reach about every expert anyway (decode batches) take the dense form
-    instead: all experts on all rows in one up GEMM, one activation pass and one batched down GEMM on the
-    stacked weights, the unchosen experts weighted by zero; that form has no host synchronisation and a
-    quarter of the launches.  Longer steps run one pair of GEMMs per expert.  (A third form, all experts as one
+    instead: all experts on all rows in one up GEMM, one activation pass that multiplies every expert's activations by
+    its routing weight (zero for the unchosen ones), and one down GEMM over all experts' activations side by side,
+    which is the weighted sum; that form has no host synchronisation and a quarter of the launches.  Longer steps run one pair of GEMMs per expert.  (A third form, all experts as one
     batch of equal-sized segments through two batched GEMMs on the stacked weights, is written and agrees with
     the others on the CPU and on small GPU steps, but a 2048-token step through it ended in a GPU memory fault
     whose cause is not found: ``BATCHED`` keeps it off on GPUs.)  The shared expert's up projection carries ``side`` extra output rows (with a
@@ -254,7 +255,7 @@ class BiasedSoftmaxMoE(nn.Module):
 
     def __init__(self, width: int, ff: int, experts: int, top: int, act: str = "relu2", shared_ff: int = 0,
                  side: int = 0, groups: int = 1, keep: int = 1, renorm: bool = True, identity: int = 0,
-                 shared_gate: bool = False, device=None, dtype=None):
+                 shared_gate: bool = False, select_bias: bool = True, device=None, dtype=None):
         super().__init__()
         n = experts + identity
         if not (0 < top <= n):
@@ -271,9 +272,9 @@ class BiasedSoftmaxMoE(nn.Module):
         kw = dict(device=device, dtype=dtype)
         f32 = dict(device=device, dtype=torch.float32)
         self.w_router = nn.Parameter(torch.empty(n, width, **f32))
-        self.bias = nn.Parameter(torch.zeros(n, **f32))
+        self.bias = nn.Parameter(torch.zeros(n, **f32)) if select_bias else None
         self.w_up = nn.Parameter(torch.empty(experts, self.up_rows, width, **kw))  # stacked: expert e is w_up[e]
-        self.w_down = nn.Parameter(torch.empty(experts, width, ff, **kw))
+        self.w_down = nn.Parameter(torch.empty(width, experts * ff, **kw))  # expert e is columns [e ff, (e + 1) ff)
         self.w_sup = nn.Parameter(torch.empty(extra, width, **kw)) if extra else None
         self.b_sup = nn.Parameter(torch.zeros(extra, **kw)) if side else None
         self.w_sdown = nn.Parameter(torch.empty(width, shared_ff, **kw)) if shared_ff else None
@@ -289,7 +290,7 @@ class BiasedSoftmaxMoE(nn.Module):
 
     @property
     def experts_down(self):
-        return self.w_down.unbind(0)
+        return self.w_down.split(self.ff, 1)
 
     PAD = 64  # expert segments run in multiples of this many rows
     DENSE_ROWS = 64  # steps of at most this many rows may take the dense form
@@ -322,23 +323,30 @@ class BiasedSoftmaxMoE(nn.Module):
         both = torch.from_numpy(np.concatenate([gi, back])).to(xs.device)
         xg = xs.index_select(0, both[:E * C]).view(E, C, W)
         a = act(torch.bmm(xg, self.w_up.transpose(1, 2)).view(E * C, self.up_rows))
-        y = torch.bmm(a.view(E, C, self.ff), self.w_down.transpose(1, 2)).view(E * C, W)
+        y = torch.bmm(a.view(E, C, self.ff), self.w_down.view(W, E, self.ff).permute(1, 2, 0)).view(E * C, W)
         return y.index_select(0, both[E * C:])
 
     def forward(self, x: torch.Tensor):
         """x [T, width] -> fp32 [T, width] (and the side columns)."""
         from llmctl.ops import hybrid as hops
 
+        from .mixers import _mm_f32
+
         T = x.shape[0]
-        act = hops.swiglu_any if self.act == "swiglu" else (lambda u: hops.act_any(u, self.act))
+
+        def act(u, scale=None):
+            if self.act == "swiglu":
+                return hops.glu_act(u, "silu", scale)
+            return hops.act_any(u, self.act, scale)
+
         topi, topw = hops.bias_topk_router(torch.nn.functional.linear(x.float(), self.w_router), self.bias, self.top,
                                            self.groups, self.keep, self.renorm)
         if self._dense(T):
             E, ff, W = self.E, self.ff, x.shape[1]
-            a = act(torch.nn.functional.linear(x, self.w_up.view(E * self.up_rows, W)).view(T * E, self.up_rows))  # [T * E, ff]
-            y = torch.bmm(a.view(T, E, ff).transpose(0, 1), self.w_down.transpose(1, 2))  # [E, T, W]
             dw = torch.zeros(T, E + self.identity, dtype=torch.float32, device=x.device).scatter_(1, topi, topw)
-            out = (y.float() * dw[:, :E].t().unsqueeze(-1)).sum(0)
+            a = act(torch.nn.functional.linear(x, self.w_up.view(E * self.up_rows, W)).view(T * E, self.up_rows),
+                    dw[:, :E].reshape(T * E))
+            out = _mm_f32(a.view(T, E * ff), self.w_down)
             if self.identity:
                 out += x.float() * dw[:, E:].sum(1, keepdim=True)
         else:

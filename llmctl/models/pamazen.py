@@ -331,7 +331,7 @@ class PamazenLM(nn.Module):
                 put(ff.bias, W[f + "correction"])
             for e in range(ff.E):
                 put(ff.w_up[e], torch.cat([W[f"{f}e{e}.gate"], W[f"{f}e{e}.up"]], 0))
-                put(ff.w_down[e], W[f"{f}e{e}.down"])
+                put(ff.experts_down[e], W[f"{f}e{e}.down"])
             if ff.shared_ff:
                 put(ff.w_sup, torch.cat([W[f + "shared.gate"], W[f + "shared.up"], W[f + "shared.sg"].reshape(1, -1)], 0))
                 put(ff.w_sdown, W[f + "shared.down"])
@@ -371,7 +371,7 @@ class PamazenLM(nn.Module):
                 continue
             out[f + "router"], out[f + "correction"] = ff.w_router, ff.bias
             for e in range(ff.E):
-                out[f"{f}e{e}.gate"], out[f"{f}e{e}.up"], out[f"{f}e{e}.down"] = ff.w_up[e, :ff.ff], ff.w_up[e, ff.ff:], ff.w_down[e]
+                out[f"{f}e{e}.gate"], out[f"{f}e{e}.up"], out[f"{f}e{e}.down"] = ff.w_up[e, :ff.ff], ff.w_up[e, ff.ff:], ff.experts_down[e]
             if ff.shared_ff:
                 s = ff.shared_ff
                 out.update({f + "shared.gate": ff.w_sup[:s], f + "shared.up": ff.w_sup[s:2 * s], f + "shared.sg": ff.w_sup[2 * s:2 * s + 1],

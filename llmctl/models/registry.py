@@ -72,5 +72,14 @@ def _register_builtin() -> None:
 
     register(pamazen.ARCHITECTURE, Family(pamazen.PamazenConfig, build_pamazen, pamazen.load_pamazen))
 
+    from . import dapipel
+
+    def build_dapipel(cfg, device=None, dtype=torch.bfloat16, seed=None):
+        if seed is not None:
+            torch.manual_seed(seed)
+        return dapipel.DapipelLM(cfg, device=device, dtype=dtype)
+
+    register(dapipel.ARCHITECTURE, Family(dapipel.DapipelConfig, build_dapipel, dapipel.load_dapipel))
+
 
 _register_builtin()

@@ -10,7 +10,6 @@ at::Tensor add_layernorm_f32_(at::Tensor x, const at::Tensor& a, const c10::opti
                               const at::Tensor& bias, double eps, bool out_bf16);
 at::Tensor rmsnorm_cols(const at::Tensor& x, const at::Tensor& w, double eps, int64_t n, bool out_bf16);
 at::Tensor sigmoid_gate_mul(const at::Tensor& o, const at::Tensor& g);
-at::Tensor swiglu_any(const at::Tensor& gu);
 at::Tensor headnorm_gate(const at::Tensor& o, const at::Tensor& w, const at::Tensor& g, double eps, bool out_bf16, bool silu);
 void latent_kv_write(const at::Tensor& dkv, const at::Tensor& norm_w, double eps, const at::Tensor& pos, const at::Tensor& inv_freq,
                      int64_t rot_dims, at::Tensor cache, const at::Tensor& slots, bool interleaved, double amp);
@@ -65,7 +64,7 @@ at::Tensor gated_norm_add_norm_f32_(at::Tensor x, const at::Tensor& y, const at:
                                     const c10::optional<at::Tensor>& w_next, double eps, bool out_bf16);
 std::tuple<at::Tensor, at::Tensor> embed_rmsnorm_f32(const at::Tensor& ids, const at::Tensor& pos, const at::Tensor& table,
                                                      const at::Tensor& pos_table, const at::Tensor& w, double eps, bool out_bf16);
-at::Tensor act_any(const at::Tensor& x, int64_t kind);
+at::Tensor act_any(const at::Tensor& x, int64_t kind, const c10::optional<at::Tensor>& scale);
 at::Tensor qk_fullnorm_prep(const at::Tensor& z, int64_t H, int64_t G, int64_t dk, int64_t dv, const at::Tensor& q_norm, const at::Tensor& k_norm,
                             double eps, const at::Tensor& pos, double temp_coef, int64_t temp_every, at::Tensor cache, const at::Tensor& slots);
 at::Tensor gla_scan(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, const at::Tensor& z, const at::Tensor& z_bias,
@@ -73,6 +72,22 @@ at::Tensor gla_scan(const at::Tensor& q, const at::Tensor& k, const at::Tensor& 
                     const c10::optional<at::Tensor>& logd, bool write_out, bool write_state);
 void gla_chunk_combine(at::Tensor S, const at::Tensor& slots, const at::Tensor& start, const at::Tensor& base, const at::Tensor& loc,
                        const at::Tensor& logd, at::Tensor init);
+at::Tensor glu_act(const at::Tensor& gu, int64_t kind, const c10::optional<at::Tensor>& scale);
+std::tuple<at::Tensor, at::Tensor> add_norm_conv(const at::Tensor& x, const at::Tensor& y, const at::Tensor& w, int64_t groups, double eps,
+                                                 const at::Tensor& cw, at::Tensor state, const at::Tensor& seq_of, const at::Tensor& cu,
+                                                 const at::Tensor& start, const at::Tensor& sslot, bool carried, bool out_bf16);
+std::tuple<at::Tensor, at::Tensor> embed_norm_conv(const at::Tensor& ids, const at::Tensor& pos, const at::Tensor& table,
+                                                   const at::Tensor& pos_table, double scale, const at::Tensor& w, int64_t groups, double eps,
+                                                   const at::Tensor& cw, at::Tensor state, const at::Tensor& seq_of, const at::Tensor& cu,
+                                                   const at::Tensor& start, const at::Tensor& sslot, bool carried);
+std::tuple<at::Tensor, at::Tensor> group_norm_f32(const at::Tensor& x, const c10::optional<at::Tensor>& y, const at::Tensor& w, int64_t groups,
+                                                  double eps, bool out_bf16);
+at::Tensor mingru_scan(const at::Tensor& z, const at::Tensor& z_bias, const at::Tensor& x_bias, at::Tensor S, const at::Tensor& slots,
+                       const at::Tensor& cu, const at::Tensor& start, int64_t portions, int64_t max_q, int64_t chunk);
+void kv_rows_write(const at::Tensor& k, const at::Tensor& v, at::Tensor cache, const at::Tensor& slots, int64_t groups);
+void diff_attn(const at::Tensor& q, const at::Tensor& cache, const at::Tensor& bt, const c10::optional<at::Tensor>& cu, const at::Tensor& ctx,
+               int64_t heads, int64_t groups, int64_t dk, int64_t dv, int64_t window, double scale, const at::Tensor& lam, double post, double eps,
+               int64_t max_q, int64_t max_ctx, bool mfma, at::Tensor out);
 }  // namespace llmctl_hybrid
 
 TORCH_LIBRARY(llmctl_hybrid, m) {
@@ -81,7 +96,6 @@ TORCH_LIBRARY(llmctl_hybrid, m) {
   m.def("add_layernorm_f32_(Tensor(a!) x, Tensor a, Tensor? b, Tensor w, Tensor bias, float eps, bool out_bf16) -> Tensor");
   m.def("rmsnorm_cols(Tensor x, Tensor w, float eps, int n, bool out_bf16) -> Tensor");
   m.def("sigmoid_gate_mul(Tensor o, Tensor g) -> Tensor");
-  m.def("swiglu_any(Tensor gu) -> Tensor");
   m.def("headnorm_gate(Tensor o, Tensor w, Tensor g, float eps, bool out_bf16, bool silu=False) -> Tensor");
   m.def("latent_kv_write(Tensor dkv, Tensor norm_w, float eps, Tensor pos, Tensor inv_freq, int rot_dims, Tensor(a!) cache, Tensor slots, bool interleaved=False, float amp=1.0) -> ()");
   m.def("latent_q_assemble(Tensor q_lat, Tensor q, Tensor pos, Tensor inv_freq, int rot_dims, int dn, bool interleaved=False, float amp=1.0) -> Tensor");
@@ -105,10 +119,17 @@ TORCH_LIBRARY(llmctl_hybrid, m) {
   m.def("delta_chunk_combine(Tensor(a!) S, Tensor slots, Tensor start, Tensor base, Tensor loc, Tensor P, Tensor(b!) init) -> ()");
   m.def("gated_norm_add_norm_f32_(Tensor(a!) x, Tensor y, Tensor r, Tensor w_post, Tensor? w_next, float eps, bool out_bf16) -> Tensor");
   m.def("embed_rmsnorm_f32(Tensor ids, Tensor pos, Tensor table, Tensor pos_table, Tensor w, float eps, bool out_bf16) -> (Tensor, Tensor)");
-  m.def("act_any(Tensor x, int kind) -> Tensor");
+  m.def("act_any(Tensor x, int kind, Tensor? scale=None) -> Tensor");
   m.def("qk_fullnorm_prep(Tensor z, int H, int G, int dk, int dv, Tensor q_norm, Tensor k_norm, float eps, Tensor pos, float temp_coef, int temp_every, Tensor(a!) cache, Tensor slots) -> Tensor");
   m.def("gla_scan(Tensor q, Tensor k, Tensor v, Tensor z, Tensor z_bias, float tau, float qscale, Tensor(a!) S, Tensor slots, Tensor cu, Tensor start, Tensor(b!)? logd=None, bool write_out=True, bool write_state=True) -> Tensor");
   m.def("gla_chunk_combine(Tensor(a!) S, Tensor slots, Tensor start, Tensor base, Tensor loc, Tensor logd, Tensor(b!) init) -> ()");
+  m.def("glu_act(Tensor gu, int kind, Tensor? scale=None) -> Tensor");
+  m.def("add_norm_conv(Tensor x, Tensor y, Tensor w, int groups, float eps, Tensor cw, Tensor(a!) state, Tensor seq_of, Tensor cu, Tensor start, Tensor sslot, bool carried, bool out_bf16) -> (Tensor, Tensor)");
+  m.def("embed_norm_conv(Tensor ids, Tensor pos, Tensor table, Tensor pos_table, float scale, Tensor w, int groups, float eps, Tensor cw, Tensor(a!) state, Tensor seq_of, Tensor cu, Tensor start, Tensor sslot, bool carried) -> (Tensor, Tensor)");
+  m.def("group_norm_f32(Tensor x, Tensor? y, Tensor w, int groups, float eps, bool out_bf16) -> (Tensor, Tensor)");
+  m.def("mingru_scan(Tensor z, Tensor z_bias, Tensor x_bias, Tensor(a!) S, Tensor slots, Tensor cu, Tensor start, int portions, int max_q, int chunk) -> Tensor");
+  m.def("kv_rows_write(Tensor k, Tensor v, Tensor(a!) cache, Tensor slots, int groups) -> ()");
+  m.def("diff_attn(Tensor q, Tensor cache, Tensor bt, Tensor? cu, Tensor ctx, int heads, int groups, int dk, int dv, int window, float scale, Tensor lam, float post, float eps, int max_q, int max_ctx, bool mfma, Tensor(a!) out) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(llmctl_hybrid, CUDA, m) {
@@ -117,7 +138,6 @@ TORCH_LIBRARY_IMPL(llmctl_hybrid, CUDA, m) {
   m.impl("add_layernorm_f32_", &llmctl_hybrid::add_layernorm_f32_);
   m.impl("rmsnorm_cols", &llmctl_hybrid::rmsnorm_cols);
   m.impl("sigmoid_gate_mul", &llmctl_hybrid::sigmoid_gate_mul);
-  m.impl("swiglu_any", &llmctl_hybrid::swiglu_any);
   m.impl("headnorm_gate", &llmctl_hybrid::headnorm_gate);
   m.impl("latent_kv_write", &llmctl_hybrid::latent_kv_write);
   m.impl("latent_q_assemble", &llmctl_hybrid::latent_q_assemble);
@@ -145,4 +165,11 @@ TORCH_LIBRARY_IMPL(llmctl_hybrid, CUDA, m) {
   m.impl("softcap_", &llmctl_hybrid::softcap_);
   m.impl("delta_scan", &llmctl_hybrid::delta_scan);
   m.impl("delta_chunk_combine", &llmctl_hybrid::delta_chunk_combine);
+  m.impl("glu_act", &llmctl_hybrid::glu_act);
+  m.impl("add_norm_conv", &llmctl_hybrid::add_norm_conv);
+  m.impl("embed_norm_conv", &llmctl_hybrid::embed_norm_conv);
+  m.impl("group_norm_f32", &llmctl_hybrid::group_norm_f32);
+  m.impl("mingru_scan", &llmctl_hybrid::mingru_scan);
+  m.impl("kv_rows_write", &llmctl_hybrid::kv_rows_write);
+  m.impl("diff_attn", &llmctl_hybrid::diff_attn);
 }

@@ -3,6 +3,7 @@
 //   gated_norm_add_norm_f32_  g = y sigmoid(r); x += g / rms(g) * w_post; h = x / rms(x) * w_next, one pass per row
 //   embed_rmsnorm_f32         x = table[id] + pos_table[position] as the fp32 stream, and its first RMS norm
 //   act_any                   relu(x)^2 or the exact (erf) GELU on a column range of a wider row
+//   glu_act                   act(gate) * up of rows [gate | up] (silu or the tanh GELU), times an optional factor per row
 // All arithmetic fp32; y, r, h in the activation dtype or fp32.
 #include "hybrid_common.h"
 
@@ -91,16 +92,16 @@ __device__ __forceinline__ float act_one(float v) {
 }
 
 template <typename T, int KIND>
-__global__ void act_kernel(const T* __restrict__ x, int64_t x_st, T* __restrict__ y, int64_t rows, int F) {
+__global__ void act_kernel(const T* __restrict__ x, int64_t x_st, const float* __restrict__ scale, T* __restrict__ y, int64_t rows, int F) {
   const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= rows * F) return;
   const int64_t r = i / F;
   const int c = (int)(i - r * F);
-  stf(y + i, act_one<KIND>(ldf(x + r * x_st + c)));
+  stf(y + i, act_one<KIND>(ldf(x + r * x_st + c)) * (scale != nullptr ? scale[r] : 1.0f));
 }
 
 template <typename T, int KIND>
-__global__ void act_vec_kernel(const T* __restrict__ x, int64_t x_st, T* __restrict__ y, int64_t rows, int F) {
+__global__ void act_vec_kernel(const T* __restrict__ x, int64_t x_st, const float* __restrict__ scale, T* __restrict__ y, int64_t rows, int F) {
   constexpr int N = Vec16<T>::N;
   const int per = F / N;
   const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -109,9 +110,41 @@ __global__ void act_vec_kernel(const T* __restrict__ x, int64_t x_st, T* __restr
   const int c = (int)(i - r * per) * N;
   float v[N];
   Vec16<T>::load(x + r * x_st + c, v);
+  const float f = scale != nullptr ? scale[r] : 1.0f;
 #pragma unroll
-  for (int k = 0; k < N; ++k) v[k] = act_one<KIND>(v[k]);
+  for (int k = 0; k < N; ++k) v[k] = act_one<KIND>(v[k]) * f;
   Vec16<T>::store(y + r * F + c, v);
+}
+
+// The tanh GELU 0.5 z (1 + tanh(y)) is z sigmoid(2 y), y = sqrt(2 / pi) (z + 0.044715 z^3).
+template <int KIND>
+__device__ __forceinline__ float gate_act(float z) {
+  const float e = KIND == 0 ? z : 1.5957691216057308f * (z + 0.044715f * z * z * z);
+  return z / (1.0f + expf(-e));
+}
+
+// gu [rows, 2F] = [gate | up] -> y [rows, F] = act(gate) up (times scale[row]); N elements a thread
+template <typename T, int KIND, int N>
+__global__ __launch_bounds__(256) void glu_act_kernel(const T* __restrict__ gu, int64_t gu_st, const float* __restrict__ scale, T* __restrict__ y,
+                                                      int64_t rows, int F) {
+  const int per = F / N;
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= rows * per) return;
+  const int64_t r = i / per;
+  const int c = (int)(i - r * per) * N;
+  float g[N], u[N];
+  if constexpr (N == 1) {
+    g[0] = ldf(gu + r * gu_st + c);
+    u[0] = ldf(gu + r * gu_st + F + c);
+  } else {
+    Vec16<T>::load(gu + r * gu_st + c, g);
+    Vec16<T>::load(gu + r * gu_st + F + c, u);
+  }
+  const float f = scale != nullptr ? scale[r] : 1.0f;
+#pragma unroll
+  for (int k = 0; k < N; ++k) g[k] = gate_act<KIND>(g[k]) * u[k] * f;
+  if constexpr (N == 1) stf(y + r * F + c, g[0]);
+  else Vec16<T>::store(y + r * F + c, g);
 }
 
 // z [T, >= H*dk + G*dk + G*dv] = [q | k | v | ...]: unit RMS over all of q and over all of k, times the weights;
@@ -208,8 +241,10 @@ std::tuple<at::Tensor, at::Tensor> embed_rmsnorm_f32(const at::Tensor& ids, cons
   return {x, h};
 }
 
-at::Tensor act_any(const at::Tensor& x, int64_t kind) {
+at::Tensor act_any(const at::Tensor& x, int64_t kind, const c10::optional<at::Tensor>& scale) {
   check_rows(x, "x");
+  if (scale.has_value()) HYB_CHECK(f32w(*scale, x.size(0)), "row factors: fp32 [rows]");
+  const float* sp = scale.has_value() ? scale->data_ptr<float>() : nullptr;
   HYB_CHECK(kind == 0 || kind == 1, "activation kind: 0 = squared relu, 1 = erf gelu");
   c10::DeviceGuard guard(x.device());
   const int64_t rows = x.size(0);
@@ -224,11 +259,39 @@ at::Tensor act_any(const at::Tensor& x, int64_t kind) {
     const int64_t nv = vec ? n / Vec16<T>::N : n;
     const dim3 grid((unsigned)((nv + 255) / 256));
     if (vec) {
-      if (kind == 0) act_vec_kernel<T, 0><<<grid, 256, 0, st>>>((const T*)x.data_ptr(), x.stride(0), (T*)y.data_ptr(), rows, F);
-      else act_vec_kernel<T, 1><<<grid, 256, 0, st>>>((const T*)x.data_ptr(), x.stride(0), (T*)y.data_ptr(), rows, F);
+      if (kind == 0) act_vec_kernel<T, 0><<<grid, 256, 0, st>>>((const T*)x.data_ptr(), x.stride(0), sp, (T*)y.data_ptr(), rows, F);
+      else act_vec_kernel<T, 1><<<grid, 256, 0, st>>>((const T*)x.data_ptr(), x.stride(0), sp, (T*)y.data_ptr(), rows, F);
     } else {
-      if (kind == 0) act_kernel<T, 0><<<grid, 256, 0, st>>>((const T*)x.data_ptr(), x.stride(0), (T*)y.data_ptr(), rows, F);
-      else act_kernel<T, 1><<<grid, 256, 0, st>>>((const T*)x.data_ptr(), x.stride(0), (T*)y.data_ptr(), rows, F);
+      if (kind == 0) act_kernel<T, 0><<<grid, 256, 0, st>>>((const T*)x.data_ptr(), x.stride(0), sp, (T*)y.data_ptr(), rows, F);
+      else act_kernel<T, 1><<<grid, 256, 0, st>>>((const T*)x.data_ptr(), x.stride(0), sp, (T*)y.data_ptr(), rows, F);
+    }
+  });
+  return y;
+}
+
+// kind: 0 = silu, 1 = tanh GELU
+at::Tensor glu_act(const at::Tensor& gu, int64_t kind, const c10::optional<at::Tensor>& scale) {
+  check_rows(gu, "gu");
+  HYB_CHECK(gu.size(1) % 2 == 0 && (kind == 0 || kind == 1), "gu: [rows, 2F]; kind: 0 = silu, 1 = tanh gelu");
+  const int64_t rows = gu.size(0);
+  const int F = (int)(gu.size(1) / 2);
+  if (scale.has_value()) HYB_CHECK(f32w(*scale, rows), "row factors: fp32 [rows]");
+  c10::DeviceGuard guard(gu.device());
+  at::Tensor y = at::empty({rows, F}, gu.options());
+  if (y.numel() == 0) return y;
+  const float* sp = scale.has_value() ? scale->data_ptr<float>() : nullptr;
+  dispatch_act(gu, [&](auto* tag) {
+    using T = std::remove_pointer_t<decltype(tag)>;
+    constexpr int N = Vec16<T>::N;
+    const bool vec = F % N == 0 && aligned16<T>(gu);
+    const dim3 grid((unsigned)((y.numel() / (vec ? N : 1) + 255) / 256));
+    auto go = [&](auto kern) { kern<<<grid, 256, 0, cur_stream()>>>((const T*)gu.data_ptr(), gu.stride(0), sp, (T*)y.data_ptr(), rows, F); };
+    if (vec) {
+      if (kind == 0) go(glu_act_kernel<T, 0, N>);
+      else go(glu_act_kernel<T, 1, N>);
+    } else {
+      if (kind == 0) go(glu_act_kernel<T, 0, 1>);
+      else go(glu_act_kernel<T, 1, 1>);
     }
   });
   return y;

@@ -154,16 +154,6 @@ __global__ void gate_mul_kernel(const TO* __restrict__ o, const TG* __restrict__
   stf(y + i, ldf(o + i) * (1.0f / (1.0f + expf(-gv))));
 }
 
-template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ y, int64_t rows, int F) {
-  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= rows * F) return;
-  const int64_t r = i / F;
-  const int c = (int)(i - r * F);
-  const float g = ldf(gu + r * 2 * F + c), u = ldf(gu + r * 2 * F + F + c);
-  stf(y + i, g / (1.0f + expf(-g)) * u);
-}
-
 // o [T, H, dv] fp32 -> y [T, H*dv]: o / rms(o over dv) * w * sigmoid(g) (silu: * g sigmoid(g)); one wave per (token, head).
 template <typename T>
 __global__ __launch_bounds__(NT) void headnorm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w,
@@ -270,20 +260,6 @@ at::Tensor sigmoid_gate_mul(const at::Tensor& o, const at::Tensor& g) {
     using T = std::remove_pointer_t<decltype(tag)>;
     gate_mul_kernel<T, T><<<dim3((unsigned)((n + 255) / 256)), 256, 0, cur_stream()>>>((const T*)o.data_ptr(), (const T*)g.data_ptr(),
                                                                                      g.stride(0), (T*)y.data_ptr(), o.size(0), (int)o.size(1), (int)(o.size(1) / g.size(1)));
-  });
-  return y;
-}
-
-at::Tensor swiglu_any(const at::Tensor& gu) {
-  HYB_CHECK(gu.is_cuda() && gu.is_contiguous() && gu.dim() == 2 && gu.size(1) % 2 == 0, "gu: contiguous [T, 2F]");
-  c10::DeviceGuard guard(gu.device());
-  const int F = (int)(gu.size(1) / 2);
-  at::Tensor y = at::empty({gu.size(0), F}, gu.options());
-  const int64_t n = y.numel();
-  if (n == 0) return y;
-  dispatch_act(gu, [&](auto* tag) {
-    using T = std::remove_pointer_t<decltype(tag)>;
-    swiglu_kernel<T><<<dim3((unsigned)((n + 255) / 256)), 256, 0, cur_stream()>>>((const T*)gu.data_ptr(), (T*)y.data_ptr(), gu.size(0), F);
   });
   return y;
 }

@@ -1,8 +1,9 @@
 """Ops of the hybrid sequence mixers: latent attention (compressed K/V cache, sliding window,
 softmax sink), grouped attention over paged rows (softmax or sigmoid weights, distance penalty), the
-mLSTM matrix memory, gated linear attention, the generalized delta rule, the group-limited sigmoid router and the
-softmax router with a selection bias (optionally group-limited), and the fp32 residual stream of parallel layers, of
-layers with a gated residual between two norms, and of layers over several residual streams (hyper-connections).
+mLSTM matrix memory, gated linear attention, the generalized delta rule, differential attention, the minGRU
+recurrence, the group-limited sigmoid router and the softmax router with a selection bias (optionally group-limited), and
+the fp32 residual stream of parallel layers, of layers with a gated residual between two norms, of layers over several
+residual streams (hyper-connections), and of layers whose sublayers read a causally convolved, group-normed input.
 
 GPU tensors run the HIP kernels of ``csrc/hybrid`` (``torch.ops.llmctl_hybrid.*``, library
 ``_llmctl_hybrid.so``); CPU tensors run :mod:`llmctl.ops.ref_hybrid`.  All activations are
@@ -249,9 +250,16 @@ def group_topk_router(logits, top: int, groups: int, keep: int):
 
 def swiglu_any(gu):
     """``silu(gate) * up`` of ``gu [..., 2F]`` = ``[gate | up]``, bf16 or fp32."""
+    return glu_act(gu, "silu")
+
+
+def glu_act(gu, kind: str, scale=None):
+    """``act(gate) * up`` of ``gu [rows, 2F]`` = ``[gate | up]`` (row-strided views allowed), bf16 or fp32, computed
+    in fp32; ``kind``: ``silu`` or ``gelu_tanh`` (the tanh form of the GELU); ``scale`` (fp32 ``[rows]``): a factor
+    per row."""
     if use_native(gu):
-        return native_hybrid().swiglu_any(gu.contiguous())
-    return ref.swiglu_any(gu)
+        return native_hybrid().glu_act(gu, {"silu": 0, "gelu_tanh": 1}[kind], scale)
+    return ref.glu_act(gu, kind, scale)
 
 
 def gated_norm_add_norm_f32_(x, y, r, w_post, w_next, eps: float, out_dtype):
@@ -353,12 +361,12 @@ def bias_topk_router(logits, bias, top: int, groups: int = 1, keep: int = 1, ren
     return ref.bias_topk_router(logits, bias, top, groups, keep, renorm)
 
 
-def act_any(x, kind: str):
+def act_any(x, kind: str, scale=None):
     """Elementwise activation of ``x`` (bf16 or fp32, computed in fp32): ``relu2`` = relu(x)^2, ``gelu`` = the
-    exact (erf) GELU."""
+    exact (erf) GELU; ``scale`` (fp32 ``[rows]``): a factor per row."""
     if use_native(x):
-        return native_hybrid().act_any(x, {"relu2": 0, "gelu": 1}[kind])
-    return ref.act_any(x, kind)
+        return native_hybrid().act_any(x, {"relu2": 0, "gelu": 1}[kind], scale)
+    return ref.act_any(x, kind, scale)
 
 
 def hc_embed_norm(ids, table, streams: int, c_in, g, eps: float, out_dtype):
@@ -450,3 +458,104 @@ def gated_add_f32_(out, y, g):
         native_hybrid().gated_add_f32_(out, y, g)
         return out
     return ref.gated_add_f32_(out, y, g)
+
+
+def _norm_conv_fits(W: int, groups: int, taps: int) -> bool:
+    """The one-pass form: 2 to 4 taps, groups of whole column quads, rows up to 8192 wide."""
+    return 2 <= taps <= 4 and W % groups == 0 and (W // groups) % 4 == 0 and W <= 8192
+
+
+def _conv_of_normed(h, cw, state, b, out_dtype):
+    """``h + conv(h)`` of an fp32 h (the second half of the unfused form)."""
+    return causal_conv(h, cw, state, b.seq_of, b.cu, b.start, b.state, True, max_len=max(b.max_q, 1 if h.shape[0] > b.Tp else 0)).to(out_dtype)
+
+
+def group_norm_f32(x, y, w, groups: int, eps: float, out_dtype):
+    """``x + y`` (``y`` None: x) of the fp32 residual stream ``[T, W]``, and its RMS norm in ``groups`` equal
+    consecutive parts, each over its own root mean square, the whole times ``w [W]`` -> ``out_dtype``."""
+    if use_native(x):
+        xo, h = native_hybrid().group_norm_f32(x, y, w, groups, eps, out_dtype == torch.bfloat16)
+        return (xo if y is not None else x), h
+    return ref.group_norm_f32(x, y, w, groups, eps, out_dtype)
+
+
+def add_norm_conv(x, y, w, groups: int, eps: float, cw, state, b, out_dtype):
+    """A sublayer's result into the fp32 residual stream and the next sublayer's input in one pass:
+    ``x <- x + y``; ``h = norm(x)`` in ``groups`` equal parts (:func:`group_norm_f32`); the result is ``h_t + sum_j cw[j]
+    h_(t - taps + 1 + j)`` per sequence and channel (``cw`` fp32, tap-major ``[taps, W]``) -> ``out_dtype``.
+    ``state`` (fp32 ``[slots, taps - 1, W]``) carries the last ``taps - 1`` rows of h of every live sequence between
+    steps; h is not rounded before the convolution.  ``b``: the step (:class:`~llmctl.models.mixers.StepBatch`).
+    Returns (the new stream, the input); ``x`` itself is left as it was."""
+    if use_native(x):
+        if _norm_conv_fits(x.shape[1], groups, cw.shape[0]):
+            return native_hybrid().add_norm_conv(x, y, w, groups, eps, cw, state, b.seq_of, b.cu, b.start, b.state,
+                                                 b.carried, out_dtype == torch.bfloat16)
+        x, h = group_norm_f32(x, y, w, groups, eps, torch.float32)
+        return x, _conv_of_normed(h, cw, state, b, out_dtype)
+    x, h = ref.group_norm_f32(x, y, w, groups, eps, torch.float32)
+    return x, ref.causal_conv(h, cw, state, b.seq_of, b.cu, b.start, b.state, True).to(out_dtype)
+
+
+def embed_norm_conv(table, pos_table, scale: float, w, groups: int, eps: float, cw, state, b):
+    """The start of the stream, ``x = table[id] * scale + pos_table[position]`` (fp32), and the first sublayer's input
+    as in :func:`add_norm_conv` (in the tables' dtype).  Returns (x, input)."""
+    if use_native(table):
+        if _norm_conv_fits(table.shape[1], groups, cw.shape[0]):
+            return native_hybrid().embed_norm_conv(b.ids, b.pos, table, pos_table, scale, w, groups, eps, cw, state,
+                                                   b.seq_of, b.cu, b.start, b.state, b.carried)
+        x = table[b.ids].float() * scale + pos_table[b.pos.long()].float()
+        _, h = group_norm_f32(x, None, w, groups, eps, torch.float32)
+        return x, _conv_of_normed(h, cw, state, b, table.dtype)
+    x = table[b.ids].float() * scale + pos_table[b.pos.long()].float()
+    _, h = ref.group_norm_f32(x, None, w, groups, eps, torch.float32)
+    return x, ref.causal_conv(h, cw, state, b.seq_of, b.cu, b.start, b.state, True).to(table.dtype)
+
+
+MINGRU_CHUNK = 32  # tokens per chunk of the chunk-parallel scan; portions of >= 2 chunks take it
+MINGRU_MAX_CHUNKS = 64  # longer portions get longer chunks
+
+
+def mingru_scan(z, z_bias, x_bias, S, b, chunk: int = 0):
+    """The minGRU recurrence over the step's tokens with its output gate: rows ``z [T, >= 3 W]`` = ``[z | x | g]``,
+    ``zeta = sigmoid(z + z_bias)``, ``u = x + x_bias``, ``cand = u + 1/2`` where ``u >= 0`` and ``sigmoid(u)`` elsewhere,
+    ``S_t = (1 - zeta) S_(t-1) + zeta cand``; returns ``S_t silu(g)`` ``[T, W]`` in z's dtype.  Everything is fp32 inside;
+    the pool ``S`` (fp32 ``[slots, W]``) is updated in place at ``b.state`` (a sequence that starts at position 0
+    begins from zeros).  Long portions run in chunks side by side: a chunk maps the state by ``S -> A S + B`` per
+    channel, so a first pass forms every chunk's (A, B) and a second one folds those before it and writes the outputs.
+    ``chunk`` > 0 fixes the chunk length."""
+    if use_native(z):
+        portions = b.p_ctx.shape[0] if b.p_ctx is not None else 0
+        if not chunk:
+            chunk = MINGRU_CHUNK
+            while chunk * MINGRU_MAX_CHUNKS < b.max_q:
+                chunk *= 2
+        return native_hybrid().mingru_scan(z, z_bias, x_bias, S, b.state, b.cu, b.start, portions, b.max_q, chunk)
+    return ref.mingru_scan(z, z_bias, x_bias, S, b.state, b.cu, b.start)
+
+
+def kv_rows_write(k, v, cache, slots, groups: int):
+    """Keys ``k [T, groups * kw]`` and values ``v [T, groups * vw]`` (column views allowed) to the tokens' cache rows
+    ``[groups, vw + kw] = [v | k]`` at ``slots``."""
+    if use_native(k):
+        native_hybrid().kv_rows_write(k, v, cache, slots, groups)
+    else:
+        ref.kv_rows_write(k, v, cache, slots, groups)
+
+
+def diff_attention(q, cache, bt, cu, ctx, heads: int, groups: int, dk: int, dv: int, window: int, scale: float, lam,
+                   post: float, eps: float, out, max_q: int = 1, max_ctx: int = 0, mfma: bool = True):
+    """Differential attention over a paged row cache.  A token's row holds ``groups`` sub-rows ``[v (dv) | k_1 (dk) |
+    k_2 (dk)]``; query rows are ``[heads, 2, dk]`` (the first columns of ``q``, row-strided views allowed) and head h
+    reads sub-row ``h // (heads // groups)``.  Map m is an ordinary softmax attention of scores ``q_m . k_m * scale`` over the
+    keys inside the causal ``window`` (i - j < window; :data:`NO_LIMIT`: plain causal); with the maps' outputs ``a_1, a_2``
+    a head gives ``o = a_1 - lam a_2`` (``lam``: fp32, one number), then ``post * o / sqrt(mean(o^2) + eps)`` over its dv
+    values, written to ``out [rows, heads * dv]``.  ``cu`` given: portions, sequence n's rows ``[cu[n], cu[n+1])`` end at
+    position ``ctx[n] - 1`` and the longest has ``max_q``; ``cu`` None: one row per sequence at ``ctx[n] - 1`` (``max_ctx``:
+    the longest context if the host knows it).  ``mfma=False`` forces the generic fp32-SIMT kernel, which also serves
+    fp32 and shapes that do not fit the matrix cores."""
+    if use_native(q):
+        native_hybrid().diff_attn(q, cache, bt, cu, ctx, heads, groups, dk, dv, window, scale, lam, post, eps, max_q, max_ctx,
+                                  mfma, out)
+    else:
+        ref.diff_attention(q, cache, bt, cu, ctx, heads, groups, dk, dv, window, scale, lam, post, eps, out)
+    return out

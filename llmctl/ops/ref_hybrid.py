@@ -248,10 +248,17 @@ def group_topk_router(logits, top, groups, keep):
     return idx, s.gather(1, idx)
 
 
-def swiglu_any(gu):
+def glu_act(gu, kind, scale=None):
     f = gu.shape[-1] // 2
     g, u = gu[..., :f].float(), gu[..., f:].float()
-    return (g * torch.sigmoid(g) * u).to(gu.dtype)
+    if kind == "silu":
+        a = g * torch.sigmoid(g)
+    elif kind == "gelu_tanh":
+        a = torch.nn.functional.gelu(g, approximate="tanh")
+    else:
+        raise ValueError(f"unknown activation {kind!r}")
+    y = a * u
+    return (y if scale is None else y * scale[:, None]).to(gu.dtype)
 
 
 def gated_norm_add_norm_f32_(x, y, r, w_post, w_next, eps, out_dtype):
@@ -321,7 +328,7 @@ def bias_topk_router(logits, bias, top, groups=1, keep=1, renorm=True):
     return idx, (w / (w.sum(-1, keepdim=True) + 1e-20) if renorm else w)
 
 
-def act_any(x, kind):
+def act_any(x, kind, scale=None):
     xf = x.float()
     if kind == "relu2":
         y = torch.relu(xf).pow(2)
@@ -329,7 +336,7 @@ def act_any(x, kind):
         y = 0.5 * xf * (1.0 + torch.erf(xf * 0.7071067811865476))
     else:
         raise ValueError(f"unknown activation {kind!r}")
-    return y.to(x.dtype)
+    return (y if scale is None else y * scale[:, None]).to(x.dtype)
 
 
 def hc_embed_norm(ids, table, streams, c_in, g, eps, out_dtype):
@@ -395,3 +402,69 @@ def softcap_(x, cap):
 def gated_add_f32_(out, y, g):
     out += y.float() * torch.sigmoid(g.float())
     return out
+
+
+def group_norm_f32(x, y, w, groups, eps, out_dtype):
+    if y is not None:
+        x = x + y.float()
+    p = x.view(x.shape[0], groups, -1)
+    h = (p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)).reshape(x.shape)
+    return x, (h * w.float()).to(out_dtype)
+
+
+def mingru_scan(z, z_bias, x_bias, S, state_slots, cu, start):
+    """Token by token; the pool S [slots, W] is read at ``state_slots[seq]`` (zeros when the sequence starts at
+    position 0) and written back after the sequence's last token of this step."""
+    W = S.shape[1]
+    zeta = torch.sigmoid(z[:, :W].float() + z_bias)
+    keep = torch.sigmoid(-(z[:, :W].float() + z_bias))
+    u = z[:, W:2 * W].float() + x_bias
+    add = zeta * torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    out = torch.zeros(z.shape[0], W, dtype=torch.float32)
+    cu_l = [int(x) for x in cu]
+    for s in range(len(cu_l) - 1):
+        if cu_l[s] == cu_l[s + 1]:
+            continue
+        slot = int(state_slots[s])
+        st = torch.zeros(W) if int(start[s]) == 0 else S[slot].clone()
+        for t in range(cu_l[s], cu_l[s + 1]):
+            st = keep[t] * st + add[t]
+            out[t] = st
+        S[slot] = st
+    g = z[:, 2 * W:3 * W].float()
+    return (out * g * torch.sigmoid(g)).to(z.dtype)
+
+
+def kv_rows_write(k, v, cache, slots, groups):
+    T = k.shape[0]
+    row = torch.cat([v.reshape(T, groups, -1), k.reshape(T, groups, -1)], -1).reshape(T, -1).to(cache.dtype)
+    ok = slots >= 0
+    cache.view(-1, cache.shape[-1])[slots[ok]] = row[ok]
+
+
+def diff_attention(q, cache, bt, cu, ctx, heads, groups, dk, dv, window, scale, lam, post, eps, out):
+    """Two softmax maps over the same values per head (cache sub-rows [v | k_1 | k_2]), ``a_1 - lam a_2``, unit RMS
+    over the values times ``post``; written to ``out``."""
+    n_rows = q.shape[0]
+    cu_l = [int(c) for c in cu] if cu is not None else list(range(n_rows + 1))
+    bs, rs = cache.shape[1], dv + 2 * dk
+    flat = cache.view(-1, groups, rs)
+    qm = q[:, :heads * 2 * dk].float().reshape(n_rows, heads, 2, dk)
+    o = torch.zeros(n_rows, heads, dv)
+    for n in range(len(cu_l) - 1):
+        a, b = cu_l[n], cu_l[n + 1]
+        if a == b:
+            continue
+        end = int(ctx[n])
+        p0 = end - (b - a)
+        kpos = torch.arange(max(0, p0 - window + 1), end)
+        rows = flat[bt[n, (kpos // bs).long()].long() * bs + kpos % bs].float().repeat_interleave(heads // groups, 1)
+        d = torch.arange(p0, end)[:, None] - kpos[None, :]
+        hide = ~((d >= 0) & (d < window))
+        m = []
+        for i in range(2):
+            s = torch.einsum("thd,khd->htk", qm[a:b, :, i], rows[:, :, dv + i * dk:dv + (i + 1) * dk]) * scale
+            m.append(torch.einsum("htk,khd->thd", torch.softmax(s.masked_fill(hide, float("-inf")), -1), rows[:, :, :dv]))
+        o[a:b] = m[0] - lam.float().reshape(()) * m[1]
+    o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * post
+    out.copy_(o.reshape(n_rows, heads * dv).to(out.dtype))

@@ -231,6 +231,7 @@ class InferenceEngine:
                           d_bt=i32(dp["bt"]) if Td else None, cu=i32(cu), start=i32(start), state=i32(state),
                           max_q=max((b - a for a, b in zip(p_cu[:-1], p_cu[1:])), default=0), cu_host=cu,
                           seq_of=i32(seq_of), d_max_ctx=int(max(dp["ctx"])) if Td else 0,
+                          carried=any(int(v) > 0 and b - a > 1 for v, a, b in zip(start, p_cu[:-1], p_cu[1:])),
                           fresh=Td == 0 and all(int(v) == 0 for v in start))
         if rows is None:
             rows = (list(pp["last"]) if Tp else []) + list(range(Tp, Tp + Td))
