@@ -69,6 +69,10 @@ def parse():
                     help="instead of the training benchmark: serving prefill / decode throughput of Malinex "
                          "configurations beside Lenitar at equal size (comma-separated sizes of "
                          "llmctl.benchmarks.hybrid.MALINEX_SIZES, or 'all'); one JSON line per size")
+    ap.add_argument("--dapipel-compare", default=None, metavar="SIZES",
+                    help="instead of the training benchmark: serving prefill / decode throughput of Dapipel "
+                         "configurations beside Malinex at equal size (comma list of "
+                         "llmctl.benchmarks.hybrid.DAPIPEL_SIZES, or 'all'); one JSON line per size")
     ap.add_argument("--pamazen-compare", default=None, metavar="SIZES",
                     help="instead of the training benchmark: serving prefill / decode throughput of Pamazen "
                          "configurations beside Malinex at equal size (comma-separated sizes of "
@@ -79,7 +83,9 @@ def parse():
 def hybrid_compare(args) -> None:
     from llmctl.benchmarks import hybrid
 
-    if args.pamazen_compare:
+    if args.dapipel_compare:
+        table, which, family = hybrid.DAPIPEL_SIZES, args.dapipel_compare, "dapipel"
+    elif args.pamazen_compare:
         table, which, family = hybrid.PAMAZEN_SIZES, args.pamazen_compare, "pamazen"
     elif args.malinex_compare:
         table, which, family = hybrid.MALINEX_SIZES, args.malinex_compare, "malinex"
@@ -94,7 +100,7 @@ def hybrid_compare(args) -> None:
 
 def main():
     args = parse()
-    if args.hybrid_compare or args.dumalix_compare or args.malinex_compare or args.pamazen_compare:
+    if args.hybrid_compare or args.dumalix_compare or args.malinex_compare or args.pamazen_compare or args.dapipel_compare:
         return hybrid_compare(args)
     import torch
     import torch.distributed as dist

@@ -6,7 +6,9 @@ closest existing model: recurrent-state layers among attention layers, routed ex
 stream) at equal width, depth, heads, experts and expert size, and of a Pamazen configuration beside Malinex (the
 closest existing model: grouped-query attention over paged rows beside a decayed matrix memory in state slots,
 softmax-routed experts with a shared one, an fp32 residual stream) at equal width, depth, heads, kv heads, experts
-and expert size.
+and expert size, and of a Dapipel configuration beside Malinex (the closest existing model: a recurrence over state
+slots in two layers of three, grouped-query attention over paged rows in the third, learned positions) at equal width,
+depth, heads, kv heads and feed-forward.
 
 Both run through the same engine calls: one prompt portion per sequence (``InferenceEngine.prefill``)
 and then one-token decode steps of the whole batch (``InferenceEngine.decode``); random weights,
@@ -58,6 +60,28 @@ PAMAZEN_SIZES = {
     "medium": dict(width=2048, layers=6, heads=16, kv_heads=4, head_dim=128, experts=8, top=2, ff=1024, window=1024, prompt=2048, batch=16),
     "large": dict(width=4096, layers=6, heads=32, kv_heads=8, head_dim=128, experts=8, top=2, ff=2048, window=1024, prompt=4096, batch=16),
 }
+
+
+# Dapipel: width, layers (every third is windowed differential attention, the others minGRU of the same width), heads of
+# ``head_dim`` (two maps of half that), kv heads, routed gated experts (``experts`` 0: a dense gated feed-forward of ``ff``,
+# beside Malinex' ungated one of 3/2 that, i.e. as many weights), window, prompt, decode batch
+DAPIPEL_SIZES = {
+    "tiny": dict(width=128, layers=3, heads=4, kv_heads=2, head_dim=32, experts=4, top=2, ff=64, window=32, prompt=64, batch=2),
+    "small": dict(width=1024, layers=6, heads=8, kv_heads=2, head_dim=128, experts=8, top=2, ff=512, window=1024, prompt=2048, batch=16),
+    "medium": dict(width=2048, layers=6, heads=16, kv_heads=4, head_dim=128, experts=8, top=2, ff=1024, window=1024, prompt=2048, batch=16),
+    "large": dict(width=4096, layers=6, heads=32, kv_heads=8, head_dim=128, experts=8, top=2, ff=2048, window=1024, prompt=4096, batch=16),
+    "medium-dense": dict(width=2048, layers=6, heads=16, kv_heads=4, head_dim=128, experts=0, top=0, ff=4096, window=1024, prompt=2048, batch=16),
+    "large-dense": dict(width=4096, layers=6, heads=32, kv_heads=8, head_dim=128, experts=0, top=0, ff=8192, window=1024, prompt=4096, batch=16),
+}
+
+
+def _configs_dapipel(s: Dict):
+    from llmctl.models.dapipel import dapipel_template
+    from llmctl.models.malinex import malinex_template
+
+    kw = dict(width=s["width"], layers=s["layers"], heads=s["heads"], kv_heads=s["kv_heads"], vocab=32000, every=3,
+              experts=s["experts"], top=s["top"], expert_ff=s["ff"], head_dim=s["head_dim"], max_positions=s["prompt"] + 256)
+    return dapipel_template(ff=s["ff"], window=s["window"], **kw), malinex_template(ff=3 * s["ff"] // 2, **kw)
 
 
 def _configs_pamazen(s: Dict):
@@ -178,7 +202,12 @@ def _measure(eng, prompt: int, batch: int, steps: int, warmup: int) -> Dict[str,
 def run(sizes: List[str], device: str = "auto", steps: int = 5, warmup: int = 2, family: str = "lenitar") -> List[Dict]:
     out = []
     for name in sizes:
-        if family == "pamazen":
+        if family == "dapipel":
+            s = DAPIPEL_SIZES[name]
+            hy, tr = _configs_dapipel(s)
+            row = {"size": name, **s}
+            pair = (("dapipel", hy), ("malinex", tr))
+        elif family == "pamazen":
             s = PAMAZEN_SIZES[name]
             hy, tr = _configs_pamazen(s)
             row = {"size": name, **s}

@@ -246,7 +246,7 @@ void launch_norm_conv(NormConvArgs a, int taps, const at::Tensor& table_or_y, bo
                       const at::Tensor& like) {
   const int quads = a.W / 4;
   // rows per workgroup: enough workgroups to fill the chip first, then fewer rows normed twice at the borders
-  a.L = std::max(1, std::min(8, a.T / 256));
+  a.L = std::max(1, std::min(8, a.T / 512));
   const int g4 = a.gs / 4;
   a.unit = 1;
   while (a.unit < 64 && g4 % (a.unit * 2) == 0) a.unit *= 2;
@@ -265,8 +265,8 @@ void launch_norm_conv(NormConvArgs a, int taps, const at::Tensor& table_or_y, bo
     auto by_taps = [&](auto tp) {
       constexpr int TAPS = decltype(tp)::value;
       if (quads <= 256) norm_conv_kernel<TY, TH, EMB, TAPS, 1, 256><<<grid, 256, lds, st>>>(a);
-      else if (quads <= 512) norm_conv_kernel<TY, TH, EMB, TAPS, 2, 256><<<grid, 256, lds, st>>>(a);
-      else if (quads <= 1024) norm_conv_kernel<TY, TH, EMB, TAPS, 2, 512><<<grid, 512, lds, st>>>(a);
+      else if (quads <= 512) norm_conv_kernel<TY, TH, EMB, TAPS, 1, 512><<<grid, 512, lds, st>>>(a);
+      else if (quads <= 1024) norm_conv_kernel<TY, TH, EMB, TAPS, 1, 1024><<<grid, 1024, lds, st>>>(a);
       else norm_conv_kernel<TY, TH, EMB, TAPS, 2, 1024><<<grid, 1024, lds, st>>>(a);
     };
     if (taps == 2) by_taps(std::integral_constant<int, 2>{});

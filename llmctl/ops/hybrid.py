@@ -512,7 +512,7 @@ def embed_norm_conv(table, pos_table, scale: float, w, groups: int, eps: float, 
 
 
 MINGRU_CHUNK = 32  # tokens per chunk of the chunk-parallel scan; portions of >= 2 chunks take it
-MINGRU_MAX_CHUNKS = 64  # longer portions get longer chunks
+MINGRU_MAX_CHUNKS = 128  # longer portions get longer chunks
 
 
 def mingru_scan(z, z_bias, x_bias, S, b, chunk: int = 0):
