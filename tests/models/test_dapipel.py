@@ -243,6 +243,42 @@ def test_heads_that_fit_the_matrix_cores(tmp_path, dev):
     check(tmp_path, dev, cfg, r, [[("a", 200), ("b", 4)]] + [[("a", 1), ("b", 1)]] * 5 + [[("a", 25)]], blocks=80)
 
 
+@pytest.mark.parametrize("seed", range(8))
+def test_random_configurations(tmp_path, dev, seed):
+    # sizes, layer order, windows, constants and schedules drawn at random (some sizes fit the vector and matrix-core
+    # forms, some do not)
+    r = random.Random(900 + seed)
+    step = r.choice([1, 4, 8])
+    size = lambda lo, hi: max(1, r.randint(lo, hi) // step) * step
+    layers = []
+    for _ in range(r.randint(2, 4)):
+        if r.random() < 0.5:
+            m = U.gru(size(4, 70))
+        else:
+            G = r.choice([1, 2, 3])
+            m = U.att(heads=G * r.choice([1, 2, 3]), kv_heads=G, dim=size(4, 40), vdim=size(4, 72), window=r.randint(1, 90),
+                      diff=r.choice([0.2, 0.5, 0.8]))
+        f = r.choice([None, U.dense(size(4, 60)), U.moe(experts=r.randint(1, 9), top=1, ff=size(4, 40))])
+        if f is not None and f["kind"] == "moe":
+            f["router"]["top"] = r.randint(1, f["router"]["experts"])
+        layers.append((m, f))
+    groups = r.choice([1, 2, 4])
+    cfg = U.config(layers, width=groups * r.choice([12, 16, 20, 33]), vocab=r.choice([37, 64, 101]), eps=r.choice([1e-6, 1e-4]), groups=groups,
+                   taps=r.choice([2, 3, 4, 5]), scale=r.choice([0.5, 2.0, 4.0]), positions=200)
+    reqs = {k: tokens(r.randint(3, 150), cfg["vocab"], 901 + i) for i, k in enumerate("abc")}
+    left, steps = {k: len(t) for k, t in reqs.items()}, []
+    while any(left.values()):
+        entries = []
+        for k in list(left):
+            if left[k] and r.random() < 0.7:
+                n = min(left[k], r.choice([1, 1, 2, 3, 17, 64, 90]))
+                entries.append((k, n))
+                left[k] -= n
+        if entries:
+            steps.append(entries)
+    check(tmp_path, dev, cfg, reqs, steps, seed=seed, blocks=40, block_size=16, bf16_all=True, bf16_tol=0.2)
+
+
 # ------------------------------------------------------------------ far keys and edges, at op level
 def _diff_case(device, dtype, bs, L, j0, form, mfma, window, H=4, G=2, dk=16, dv=24, which=0):
     """One key (position j0) stands out in map ``which`` for the last queries; they see it if it lies in their window.
