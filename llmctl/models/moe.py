@@ -247,10 +247,11 @@ class BiasedSoftmaxMoE(nn.Module):
     few tokens that between them reach about every expert anyway (decode batches) take the dense form
     instead: all experts on all rows in one up GEMM, one activation pass that multiplies every expert's activations by
     its routing weight (zero for the unchosen ones), and one down GEMM over all experts' activations side by side,
-    which is the weighted sum; that form has no host synchronisation and a quarter of the launches.  Longer steps run one pair of GEMMs per expert.  (A third form, all experts as one
-    batch of equal-sized segments through two batched GEMMs on the stacked weights, is written and agrees with
-    the others on the CPU and on small GPU steps, but a 2048-token step through it ended in a GPU memory fault
-    whose cause is not found: ``BATCHED`` keeps it off on GPUs.)  The shared expert's up projection carries ``side`` extra output rows (with a
+    which is the weighted sum; that form has no host synchronisation and a quarter of the launches.  Longer steps run one pair of GEMMs per expert.  (A third
+    form, all experts as one batch of equal-sized segments through two batched GEMMs on the stacked weights, agrees with
+    the others on the CPU and on small GPU steps, but a 2048-token step through it ended in a GPU memory fault: its right
+    operands are transposed views, a form of the batched bf16 product that has faulted on this platform.  ``BATCHED`` keeps it
+    off on GPUs.)  The shared expert's up projection carries ``side`` extra output rows (with a
     bias) that are handed back; without a shared expert they are a projection of their own."""
 
     def __init__(self, width: int, ff: int, experts: int, top: int, act: str = "relu2", shared_ff: int = 0,

@@ -541,11 +541,11 @@ void diff_attn(const at::Tensor& q, const at::Tensor& cache, const at::Tensor& b
     a.nvt = (int)((dv + NDBv * 32 - 1) / (NDBv * 32));
     HYB_CHECK(G * a.hpg * a.nvt <= 65535, "grid too large");
     at::Tensor ws_o, ws_ml;
-    if (!cu.has_value()) {  // decode: split the visible key tiles over workgroups until the launch has a few hundred
+    if (!cu.has_value()) {  // decode: split the visible key tiles over workgroups, one for every CU at most (a CU holds one)
       const int64_t span = std::min<int64_t>(a.window, max_ctx > 0 ? max_ctx : (int64_t)1 << 30);
       const int tiles = (int)std::min<int64_t>((span + PKB - 1) / PKB + 1, 1 << 20);
       const long blocks = (long)ns * G * a.hpg * a.nvt;
-      while (a.nsplit < tiles && a.nsplit < 32 && blocks * a.nsplit < 512) a.nsplit *= 2;
+      while (a.nsplit < tiles && a.nsplit < 32 && blocks * a.nsplit * 2 <= 256) a.nsplit *= 2;
     }
     if (a.nsplit > 1 || a.nvt > 1) {
       ws_o = at::empty({rows * H * a.nsplit * 2 * dv}, q.options().dtype(at::kFloat));
