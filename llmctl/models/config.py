@@ -304,6 +304,12 @@ def get_model_config(name_or_path: str) -> ModelConfig:
         kv = {p[0]: int(p[1:]) for p in key.split("-")[1:] if p[1:].isdigit()}
         return dapipel_template(width=kv.get("w", 256), layers=kv.get("l", 4), heads=kv.get("h", 4),
                                 kv_heads=kv.get("g", 2), experts=kv.get("e", 0))
+    if key.startswith("dumazen-"):  # dumazen-w<width>-l<layers>[-h<heads>][-g<kv heads>]: random-init template
+        from .dumazen import dumazen_template
+
+        kv = {p[0]: int(p[1:]) for p in key.split("-")[1:] if p[1:].isdigit()}
+        return dumazen_template(width=kv.get("w", 256), layers=kv.get("l", 4), heads=kv.get("h", 4),
+                                kv_heads=kv.get("g", 2))
     if key in ALIASES:
         t, s = ALIASES[key]
         return ModelConfig.from_dict(MODEL_TEMPLATES[t][s])

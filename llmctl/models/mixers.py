@@ -30,6 +30,9 @@
 * :class:`DeltaRule` — the generalized delta rule: a matrix memory per head that decays per key channel, removes
   what it holds along the current unit key at a learned rate and then writes ``k v^T``; low-rank decay projection
   through a ``tanh``, per-head unit RMS, weight and sigmoid gate on the read-out; state in a slot pool.
+* :class:`GatedDeltaRule`, :class:`Mamba2`, :class:`Retention` — matrix memories with one decay per head and token (from
+  the input, or fixed), the first subtracting what the memory already gives for a key before it writes; short
+  convolutions with silu ahead of the first two, rotary ahead of the third; one scan serves all three.
 * :class:`ParallelMixers` — two mixers on the same input whose results are added with fixed factors (one input GEMM
   on the stacked weights; paged rows for the one, state pools for the other).
 * :class:`MLSTM` — the xLSTM matrix memory: per head a ``[dk, dv]`` state with exponential input gate,
@@ -88,13 +91,21 @@ def rotary_frequencies(base: float, dims: int, scaling: Optional[dict] = None, d
     ``scaling`` = ``{factor, original, fast, slow}`` applies YaRN: with ``where(t) = dims ln(original /
     (2 pi t)) / (2 ln base)`` the pairs below ``floor(where(fast))`` keep their frequency, those above
     ``ceil(where(slow))`` are divided by ``factor``, a linear ramp lies between; cos and sin are multiplied
-    by ``0.1 ln(factor) + 1``.  ``scaling`` = ``{factor}`` alone is linear scaling: every frequency is divided
+    by ``0.1 ln(factor) + 1``.  ``scaling`` = ``{factor, original, low, high}`` goes by wavelength ``2 pi / f``: below ``original /
+    high`` f stays, above ``original / low`` it is divided by ``factor``, between them the two are blended by ``(original /
+    wavelength - low) / (high - low)``.  ``scaling`` = ``{factor}`` alone is linear scaling: every frequency is divided
     by ``factor``."""
     i = torch.arange(dims // 2, dtype=torch.float64)
     f = float(base) ** (-2.0 * i / max(dims, 1))
     amp = 1.0
     if scaling and "original" not in scaling:
         f = f / float(scaling.get("factor", 1.0))
+    elif scaling and "low" in scaling:
+        factor, low, high = float(scaling["factor"]), float(scaling["low"]), float(scaling["high"])
+        turns = float(scaling["original"]) * f / (2.0 * math.pi)  # original / wavelength
+        keep = ((turns - low) / max(high - low, 1e-30)).clamp(0.0, 1.0)
+        keep = torch.where(turns > high, torch.ones_like(keep), torch.where(turns < low, torch.zeros_like(keep), keep))
+        f = (1.0 - keep) * f / factor + keep * f
     elif scaling:
         factor, orig = float(scaling["factor"]), float(scaling["original"])
         where = lambda t: dims * math.log(orig / (2.0 * math.pi * t)) / (2.0 * math.log(float(base)))
@@ -253,8 +264,9 @@ class CausalConv(nn.Module):
 class GroupedAttention(nn.Module):
     """Grouped-query attention (``heads`` query heads over ``kv_heads`` key / value heads; key size
     ``dim``, value size ``vdim``) with, each optional: ``conv_taps`` short causal convolutions on the
-    projected q, k, v; ``qk_norm``: per-head RMS norm of q and k; rotary on the first ``rot_dims`` entries (YaRN
-    or linear scaling by ``rot_scaling``, neighbour pairs when ``interleaved``); ``rotate_values``: the value of position j
+    projected q, k, v; ``bias``: biases on the projections; ``qk_norm``: True = per-head RMS norm of q and k (one weight of
+    the head's size each), ``"whole"`` = one RMS norm over all of q and one over all of k ahead of the split into heads;
+    rotary on the first ``rot_dims`` entries (frequency scaling by ``rot_scaling``, neighbour pairs when ``interleaved``); ``rotate_values``: the value of position j
     is cached turned by ``j * rot_base^(-2m/vdim)`` per pair m and a head's output at position i is
     turned back by i, so the sum weighs values by their relative position; ``temperature``: a learned
     per-head factor on the scaled scores; ``softcap`` c: the scaled score becomes ``c tanh(score / c)``;
@@ -269,9 +281,9 @@ class GroupedAttention(nn.Module):
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, rot_base: float, rot_dims: int,
                  scale: float, eps: float, conv_taps: int = 0, rot_scaling: Optional[dict] = None,
                  interleaved: bool = True, rotate_values: bool = False, temperature: bool = False,
-                 chunk: Optional[int] = None, window: Optional[int] = None, sink=False, qk_norm: bool = True,
+                 chunk: Optional[int] = None, window: Optional[int] = None, sink=False, qk_norm=True,
                  values: str = "own", value_mix: Optional[str] = None, softcap: float = 0.0, keep_first: int = 0,
-                 device=None, dtype=None):
+                 bias: bool = False, device=None, dtype=None):
         super().__init__()
         if heads % kv_heads or rot_dims % 2 or rot_dims > dim:
             raise ValueError("kv heads must divide the heads; rotary dims must be even and fit the head")
@@ -281,6 +293,8 @@ class GroupedAttention(nn.Module):
             raise ValueError("values that are the keys have the keys' size and are neither turned, mixed nor convolved")
         if value_mix not in (None, "source", "mix"):
             raise ValueError("value_mix: None, 'source' or 'mix'")
+        if qk_norm == "whole" and (values != "own" or value_mix or rotate_values):
+            raise ValueError("a norm over all of q and k goes with plain values")
         self.width, self.H, self.G, self.dk, self.dv = width, heads, kv_heads, dim, vdim
         self.rot_dims, self.scale, self.eps, self.interleaved = rot_dims, scale, eps, interleaved
         self.chunk = int(chunk) if chunk else hops.NO_LIMIT
@@ -292,10 +306,12 @@ class GroupedAttention(nn.Module):
         cols = (heads + kv_heads) * dim + (0 if self.v_from_k else kv_heads * vdim)
         self.cols = cols
         self.w_qkv = nn.Parameter(torch.empty(cols, width, **kw))  # [W_q ; W_k ; W_v]: the input is read once
+        self.b_qkv = nn.Parameter(torch.zeros(cols, **kw)) if bias else None
         self.w_o = nn.Parameter(torch.empty(width, heads * vdim, **kw))
         self.conv = CausalConv(cols, conv_taps, residual=False, device=device) if conv_taps else None
-        self.q_norm = nn.Parameter(torch.ones(dim, **f32)) if qk_norm else None
-        self.k_norm = nn.Parameter(torch.ones(dim, **f32)) if qk_norm else None
+        self.whole_norm = qk_norm == "whole"
+        self.q_norm = nn.Parameter(torch.ones(heads * dim if self.whole_norm else dim, **f32)) if qk_norm else None
+        self.k_norm = nn.Parameter(torch.ones(kv_heads * dim if self.whole_norm else dim, **f32)) if qk_norm else None
         self.temp = nn.Parameter(torch.ones(heads, **f32)) if temperature else None
         if sink is True:
             self.sink = nn.Parameter(torch.zeros(heads, **f32))
@@ -322,6 +338,10 @@ class GroupedAttention(nn.Module):
     def w_in(self):
         return self.w_qkv
 
+    @property
+    def b_in(self):
+        return self.b_qkv
+
     def state_shapes(self):
         return [self.conv.state_shape()] if self.conv is not None else []
 
@@ -330,7 +350,7 @@ class GroupedAttention(nn.Module):
         rows, states = cache if isinstance(cache, tuple) else (cache, ())
         T = h.shape[0]
         if z is None:
-            z = F.linear(h, self.w_qkv)
+            z = F.linear(h, self.w_qkv, self.b_qkv)
         if self.conv is not None:
             z = self.conv(z, b, states[0])
         v_first = None
@@ -340,9 +360,13 @@ class GroupedAttention(nn.Module):
                 b.scratch[self.VALUE_SOURCE] = z[:, v0:v0 + self.G * self.dv]
             else:
                 v_first = b.scratch[self.VALUE_SOURCE]
-        q = hops.attn_qkv_prep(z, self.H, self.G, self.dk, self.dv, self.q_norm, self.k_norm, self.eps, b.pos,
-                               self.inv_freq, self.rot_dims, self.interleaved, self.rot_amp, self.v_freq, rows, b.slots,
-                               v_from_k=self.v_from_k, v_first=v_first, v_lambda=self.vmix if v_first is not None else None)
+        if self.whole_norm:
+            q = hops.qk_fullnorm_prep(z, self.H, self.G, self.dk, self.dv, self.q_norm, self.k_norm, self.eps, b.pos, 0.0, 1, rows,
+                                      b.slots, self.inv_freq, self.rot_dims, self.interleaved, self.rot_amp)
+        else:
+            q = hops.attn_qkv_prep(z, self.H, self.G, self.dk, self.dv, self.q_norm, self.k_norm, self.eps, b.pos,
+                                   self.inv_freq, self.rot_dims, self.interleaved, self.rot_amp, self.v_freq, rows, b.slots,
+                                   v_from_k=self.v_from_k, v_first=v_first, v_lambda=self.vmix if v_first is not None else None)
         opt = dict(groups=self.G, koff=self.dv, chunk=self.chunk, hscale=self.temp, ofreq=self.v_freq,
                    softcap=self.softcap, keep_first=self.keep_first)
         outs = []
@@ -535,22 +559,23 @@ class SigmoidAttention(nn.Module):
 
 
 class DenseFF(nn.Module):
-    """``W_down act(W_up h)`` with ``act`` one of :func:`llmctl.ops.hybrid.act_any`'s kinds; the up
-    projection carries ``side`` extra output rows (with a bias) that are handed back."""
+    """``W_down act(W_up h)`` with ``act`` one of :func:`llmctl.ops.hybrid.act_any`'s kinds (``bias``: both projections
+    have one); the up projection carries ``side`` extra output rows (with a bias) that are handed back."""
 
-    def __init__(self, width: int, ff: int, act: str = "gelu", side: int = 0, device=None, dtype=None):
+    def __init__(self, width: int, ff: int, act: str = "gelu", side: int = 0, bias: bool = False, device=None, dtype=None):
         super().__init__()
         self.ff, self.act, self.side = ff, act, side
         kw = dict(device=device, dtype=dtype)
         self.w_up = nn.Parameter(torch.empty(ff + side, width, **kw))
-        self.b_up = nn.Parameter(torch.zeros(ff + side, **kw)) if side else None
+        self.b_up = nn.Parameter(torch.zeros(ff + side, **kw)) if side or bias else None
         self.w_down = nn.Parameter(torch.empty(width, ff, **kw))
+        self.b_down = nn.Parameter(torch.zeros(width, **kw)) if bias else None
         _init(self.w_up, 0.02)
         _init(self.w_down, 0.02)
 
     def forward(self, h: torch.Tensor):
         z = F.linear(h, self.w_up, self.b_up)
-        y = F.linear(hops.act_any(z[:, :self.ff], self.act), self.w_down)
+        y = F.linear(hops.act_any(z[:, :self.ff], self.act), self.w_down, self.b_down)
         return (y, z[:, self.ff:]) if self.side else y
 
 
@@ -711,6 +736,155 @@ class DeltaRule(nn.Module):
         return F.linear(hops.headnorm_gate(o, self.norm, g, self.eps, h.dtype), self.w_o)
 
 
+def _rows8(n: int) -> int:
+    """Rows of a fused input weight, filled up so that every row of its product starts 16-byte aligned."""
+    return (n + 7) // 8 * 8
+
+
+def _own_states(state):
+    """The state pools of a recurrent mixer, from a layer's entry of either kind (pools, or paged rows and pools)."""
+    return state[1] if isinstance(state, tuple) and len(state) == 2 and isinstance(state[1], tuple) else state
+
+
+class GatedDeltaRule(nn.Module):
+    """The gated delta rule: per head a memory ``S [dim, vdim]`` with one decay per head and token, ``S <- g S``, ``u = beta (v -
+    S^T k)``, ``S <- S + k u^T``, ``o = S^T q``.  q, k (``kv_heads`` of them) and v pass short causal convolutions and silu;
+    q and k become unit vectors per head (``x / sqrt(sum x^2 + key_eps)``), q times ``dim^-1/2``; ``beta = sigmoid(W_b h)``, ``g =
+    exp(-exp(A_log) softplus(W_a h + dt_bias))``.  Each head's ``o`` over its root mean square, times one weight of vdim for
+    all heads, times ``silu(W_g h)``, then ``W_o``.  The fused input weight is ``[W_q ; W_k ; W_v ; W_g ; W_a ; W_b]``; state:
+    the memory (fp32) and the convolutions' last inputs."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float, key_eps: float = 1e-6,
+                 device=None, dtype=None):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("kv heads must divide the heads")
+        self.width, self.H, self.G, self.dk, self.dv, self.eps, self.key_eps = width, heads, kv_heads, dim, vdim, eps, float(key_eps)
+        kw = dict(device=device, dtype=dtype)
+        f32 = dict(device=device, dtype=torch.float32)
+        channels = 2 * kv_heads * dim + heads * vdim
+        self.cols = channels + heads * vdim + 2 * heads
+        self.w_in = nn.Parameter(torch.zeros(_rows8(self.cols), width, **kw))
+        self.conv = CausalConv(channels, taps, residual=False, device=device)
+        self.a_log = nn.Parameter(torch.zeros(heads, **f32))
+        self.dt_bias = nn.Parameter(torch.zeros(heads, **f32))
+        self.norm = nn.Parameter(torch.ones(vdim, **f32))
+        self.w_o = nn.Parameter(torch.empty(width, heads * vdim, **kw))
+        _init(self.w_in[:self.cols], 0.02)
+        _init(self.w_o, 0.02)
+        _init(self.conv.weight, 0.5)
+        self._nw = None
+
+    cache_kind = "state"
+    cache_row = 0
+
+    def state_shapes(self):
+        return [(self.H, self.dk, self.dv), self.conv.state_shape()]
+
+    _norm_rows = GatedLinearAttention._norm_rows
+
+    def step(self, h: torch.Tensor, b: StepBatch, state, z: Optional[torch.Tensor] = None) -> torch.Tensor:
+        S, carried = _own_states(state)
+        H, G, dv = self.H, self.G, self.dv
+        if z is None:
+            z = F.linear(h, self.w_in)
+        c, g0 = self.conv.channels, self.conv.channels + H * dv
+        qk, v = hops.conv_silu_unit(z[:, :c], self.conv.tap_major(), None, carried, b, G, G, self.dk, self.dk ** -0.5, self.key_eps)
+        o = hops.memory_scan(qk[:, :G], qk[:, G:], v.unflatten(1, (H, dv)), "delta", S, b, ga=z[:, g0:g0 + H],
+                             gb=z[:, g0 + H:g0 + 2 * H], a_log=self.a_log, dt_bias=self.dt_bias)
+        return F.linear(hops.headnorm_gate(o, self._norm_rows(), z[:, c:g0], self.eps, h.dtype, silu=True), self.w_o)
+
+
+class Mamba2(nn.Module):
+    """Mamba-2 (state-space duality): ``W_in h = [z | x | B | C | dt]``; x, B and C pass a short causal convolution with bias and
+    silu; ``dt = softplus(dt + dt_bias)``; per head ``S [state, vdim]``: ``S_t = exp(-exp(A_log) dt) S_(t-1) + dt B x^T``, ``y = S^T C +
+    D x`` with B and C shared by the heads of one of ``groups`` groups.  The heads are concatenated, multiplied by ``silu(z)``
+    and then RMS-normed in ``norm_groups`` equal parts, times a weight; ``W_o``.  State: the memory (fp32) and the
+    convolution's last inputs."""
+
+    def __init__(self, width: int, heads: int, vdim: int, state: int, groups: int, taps: int, norm_groups: int, eps: float,
+                 device=None, dtype=None):
+        super().__init__()
+        if heads % groups or (heads * vdim) % norm_groups:
+            raise ValueError("groups must divide the heads, norm groups the inner width")
+        self.width, self.H, self.dv, self.N, self.G, self.norm_groups, self.eps = width, heads, vdim, state, groups, norm_groups, eps
+        kw = dict(device=device, dtype=dtype)
+        f32 = dict(device=device, dtype=torch.float32)
+        self.inner = heads * vdim
+        channels = self.inner + 2 * groups * state
+        self.cols = self.inner + channels + heads
+        self.w_in = nn.Parameter(torch.zeros(_rows8(self.cols), width, **kw))
+        self.conv = CausalConv(channels, taps, residual=False, device=device)
+        self.conv_bias = nn.Parameter(torch.zeros(channels, **f32))
+        self.a_log = nn.Parameter(torch.zeros(heads, **f32))
+        self.dt_bias = nn.Parameter(torch.zeros(heads, **f32))
+        self.skip = nn.Parameter(torch.ones(heads, **f32))
+        self.norm = nn.Parameter(torch.ones(self.inner, **f32))
+        self.w_o = nn.Parameter(torch.empty(width, self.inner, **kw))
+        _init(self.w_in[:self.cols], 0.02)
+        _init(self.w_o, 0.02)
+        _init(self.conv.weight, 0.5)
+
+    cache_kind = "state"
+    cache_row = 0
+
+    def state_shapes(self):
+        return [(self.H, self.N, self.dv), self.conv.state_shape()]
+
+    def step(self, h: torch.Tensor, b: StepBatch, state) -> torch.Tensor:
+        S, carried = _own_states(state)
+        T, n = h.shape[0], self.inner
+        z = F.linear(h, self.w_in)
+        c = n + self.conv.channels
+        _, xbc = hops.conv_silu_unit(z[:, n:c], self.conv.tap_major(), self.conv_bias, carried, b, 0, 0, 0, 1.0)
+        B, C = (xbc[:, n + i * self.G * self.N:n + (i + 1) * self.G * self.N].unflatten(1, (self.G, self.N)) for i in range(2))
+        o = hops.memory_scan(C, B, xbc[:, :n].unflatten(1, (self.H, self.dv)), "ssm", S, b, ga=z[:, c:c + self.H], a_log=self.a_log,
+                             dt_bias=self.dt_bias, skip=self.skip)
+        return F.linear(hops.gate_groupnorm(o.view(T, n), z[:, :n], self.norm, self.norm_groups, self.eps, h.dtype), self.w_o)
+
+
+class Retention(nn.Module):
+    """Retention: linear attention with a fixed decay per head and neither softmax nor denominator, ``S_t = decay_h S_(t-1) + k v^T``,
+    ``o = S^T q``; rotary on q and k (half pairs unless ``interleaved``), k times ``dim^-1/2`` after it.  Each head's ``o`` over its
+    root mean square (no weight), times ``silu(W_g h)``, then ``W_o``.  The fused input weight is ``[W_q ; W_k ; W_v ; W_g]``; the
+    memory is fp32 and lives in a state slot."""
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, decay, rot_base: float, rot_dims: int, eps: float,
+                 rot_scaling: Optional[dict] = None, interleaved: bool = False, device=None, dtype=None):
+        super().__init__()
+        if len(decay) != heads or any(not 0.0 < float(d) for d in decay):
+            raise ValueError("one positive decay per head")
+        if rot_dims % 2 or rot_dims > dim:
+            raise ValueError("rotary dims must be even and fit the head")
+        self.width, self.H, self.dk, self.dv, self.eps = width, heads, dim, vdim, eps
+        self.rot_dims, self.interleaved = rot_dims, interleaved
+        kw = dict(device=device, dtype=dtype)
+        self.cols = 2 * heads * (dim + vdim)
+        self.w_in = nn.Parameter(torch.zeros(_rows8(self.cols), width, **kw))
+        self.w_o = nn.Parameter(torch.empty(width, heads * vdim, **kw))
+        _init(self.w_in[:self.cols], 0.02)
+        _init(self.w_o, 0.02)
+        inv_freq, self.rot_amp = rotary_frequencies(rot_base, rot_dims, rot_scaling, device)
+        self.register_buffer("inv_freq", inv_freq, persistent=False)
+        logs = torch.tensor([math.log(float(d)) for d in decay], dtype=torch.float32, device=device)
+        self.register_buffer("log_decay", logs, persistent=False)
+
+    cache_kind = "state"
+    cache_row = 0
+
+    def state_shapes(self):
+        return [(self.H, self.dk, self.dv)]
+
+    def step(self, h: torch.Tensor, b: StepBatch, state) -> torch.Tensor:
+        S = _own_states(state)[0]
+        H, dk, dv = self.H, self.dk, self.dv
+        z = F.linear(h, self.w_in)
+        qk = hops.rotary_f32(z, H, H, dk, b.pos, self.inv_freq, self.rot_dims, self.interleaved, self.rot_amp, dk ** -0.5)
+        v0, g0 = 2 * H * dk, 2 * H * dk + H * dv
+        o = hops.memory_scan(qk[:, :H], qk[:, H:], z[:, v0:g0].unflatten(1, (H, dv)), "fixed", S, b, log_decay=self.log_decay)
+        return F.linear(hops.headnorm_gate(o, None, z[:, g0:g0 + H * dv], self.eps, h.dtype, silu=True), self.w_o)
+
+
 class ParallelMixers(nn.Module):
     """Two mixers side by side on the same input: the result is ``left_scale * left(h) + right_scale * right(h)``.
     ``step`` returns the two results with their factors (the layer's residual pass sums them); both input
@@ -734,19 +908,27 @@ class ParallelMixers(nn.Module):
     def state_shapes(self):
         return list(self.left.state_shapes()) + list(self.right.state_shapes())
 
-    def _stacked(self) -> torch.Tensor:
-        """[W_in left ; W_in right] (made once; serving weights are static)."""
-        a, c = self.left.w_in, self.right.w_in
-        key = (a.data_ptr(), a._version, c.data_ptr(), c._version)
+    def _stacked(self):
+        """([W_in left ; W_in right], their biases or None, the right one's first row); made once, serving weights are
+        static.  Zero rows fill both up to multiples of 8, so that every row of the product starts aligned."""
+        parts = [(m.w_in, getattr(m, "b_in", None)) for m in (self.left, self.right)]
+        key = tuple((t.data_ptr(), t._version) for p in parts for t in p if t is not None)
         if self._w_key != key:
-            self._w, self._w_key = torch.cat([a.detach(), c.detach()], 0).contiguous(), key
+            ws, bs = [], []
+            for w, bias in parts:
+                n = (w.shape[0] + 7) // 8 * 8
+                ws.append(F.pad(w.detach(), (0, 0, 0, n - w.shape[0])))
+                bs.append(w.new_zeros(n) if bias is None else F.pad(bias.detach(), (0, n - w.shape[0])))
+            has_bias = any(bias is not None for _, bias in parts)
+            self._w = (torch.cat(ws, 0).contiguous(), torch.cat(bs) if has_bias else None, ws[0].shape[0])
+            self._w_key = key
         return self._w
 
     def step(self, h: torch.Tensor, b: StepBatch, cache):
         rows, states = cache
         nl = len(self.left.state_shapes())
-        z = F.linear(h, self._stacked())
-        cl = self.left.w_in.shape[0]
-        yl = self.left.step(h, b, (rows, tuple(states[:nl])), z=z[:, :cl])
-        yr = self.right.step(h, b, (rows, tuple(states[nl:])), z=z[:, cl:])
+        w, bias, c0 = self._stacked()
+        z = F.linear(h, w, bias)
+        yl = self.left.step(h, b, (rows, tuple(states[:nl])), z=z[:, :self.left.w_in.shape[0]])
+        yr = self.right.step(h, b, (rows, tuple(states[nl:])), z=z[:, c0:c0 + self.right.w_in.shape[0]])
         return (yl, self.left_scale), (yr, self.right_scale)

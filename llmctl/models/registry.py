@@ -81,5 +81,14 @@ def _register_builtin() -> None:
 
     register(dapipel.ARCHITECTURE, Family(dapipel.DapipelConfig, build_dapipel, dapipel.load_dapipel))
 
+    from . import dumazen
+
+    def build_dumazen(cfg, device=None, dtype=torch.bfloat16, seed=None):
+        if seed is not None:
+            torch.manual_seed(seed)
+        return dumazen.DumazenLM(cfg, device=device, dtype=dtype)
+
+    register(dumazen.ARCHITECTURE, Family(dumazen.DumazenConfig, build_dumazen, dumazen.load_dumazen))
+
 
 _register_builtin()

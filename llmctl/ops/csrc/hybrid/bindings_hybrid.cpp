@@ -10,7 +10,7 @@ at::Tensor add_layernorm_f32_(at::Tensor x, const at::Tensor& a, const c10::opti
                               const at::Tensor& bias, double eps, bool out_bf16);
 at::Tensor rmsnorm_cols(const at::Tensor& x, const at::Tensor& w, double eps, int64_t n, bool out_bf16);
 at::Tensor sigmoid_gate_mul(const at::Tensor& o, const at::Tensor& g);
-at::Tensor headnorm_gate(const at::Tensor& o, const at::Tensor& w, const at::Tensor& g, double eps, bool out_bf16, bool silu);
+at::Tensor headnorm_gate(const at::Tensor& o, const c10::optional<at::Tensor>& w, const at::Tensor& g, double eps, bool out_bf16, bool silu);
 void latent_kv_write(const at::Tensor& dkv, const at::Tensor& norm_w, double eps, const at::Tensor& pos, const at::Tensor& inv_freq,
                      int64_t rot_dims, at::Tensor cache, const at::Tensor& slots, bool interleaved, double amp);
 at::Tensor latent_q_assemble(const at::Tensor& q_lat, const at::Tensor& q, const at::Tensor& pos, const at::Tensor& inv_freq,
@@ -66,7 +66,8 @@ std::tuple<at::Tensor, at::Tensor> embed_rmsnorm_f32(const at::Tensor& ids, cons
                                                      const at::Tensor& pos_table, const at::Tensor& w, double eps, bool out_bf16);
 at::Tensor act_any(const at::Tensor& x, int64_t kind, const c10::optional<at::Tensor>& scale);
 at::Tensor qk_fullnorm_prep(const at::Tensor& z, int64_t H, int64_t G, int64_t dk, int64_t dv, const at::Tensor& q_norm, const at::Tensor& k_norm,
-                            double eps, const at::Tensor& pos, double temp_coef, int64_t temp_every, at::Tensor cache, const at::Tensor& slots);
+                            double eps, const at::Tensor& pos, double temp_coef, int64_t temp_every, at::Tensor cache, const at::Tensor& slots,
+                            const c10::optional<at::Tensor>& freq, int64_t rot, bool interleaved, double amp);
 at::Tensor gla_scan(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, const at::Tensor& z, const at::Tensor& z_bias,
                     double tau, double qscale, at::Tensor S, const at::Tensor& slots, const at::Tensor& cu, const at::Tensor& start,
                     const c10::optional<at::Tensor>& logd, bool write_out, bool write_state);
@@ -88,6 +89,27 @@ void kv_rows_write(const at::Tensor& k, const at::Tensor& v, at::Tensor cache, c
 void diff_attn(const at::Tensor& q, const at::Tensor& cache, const at::Tensor& bt, const c10::optional<at::Tensor>& cu, const at::Tensor& ctx,
                int64_t heads, int64_t groups, int64_t dk, int64_t dv, int64_t window, double scale, const at::Tensor& lam, double post, double eps,
                int64_t max_q, int64_t max_ctx, bool mfma, at::Tensor out);
+std::tuple<at::Tensor, at::Tensor> conv_silu_unit(const at::Tensor& u, const at::Tensor& w, const c10::optional<at::Tensor>& bias, at::Tensor state,
+                                                  const at::Tensor& seq_of, const at::Tensor& cu, const at::Tensor& start, const at::Tensor& sslot,
+                                                  int64_t nq, int64_t nk, int64_t dk, double qscale, double eps, int64_t max_len);
+using OptT = c10::optional<at::Tensor>;
+void memory_decode(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, int64_t kind, const OptT& ga, const OptT& gb, const OptT& a_log,
+                   const OptT& dt_bias, const OptT& log_decay, const OptT& skip, at::Tensor S, const at::Tensor& slots, const at::Tensor& start,
+                   at::Tensor out, int64_t row0);
+void memory_chunks(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, int64_t kind, const OptT& ga, const OptT& gb, const OptT& a_log,
+                   const OptT& dt_bias, const OptT& log_decay, const OptT& skip, at::Tensor S, const OptT& slots, const at::Tensor& cu,
+                   const OptT& start, const OptT& init, at::Tensor out, int64_t rows);
+void memory_chunk_local(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, int64_t kind, const OptT& ga, const OptT& gb, const OptT& a_log,
+                        const OptT& dt_bias, const OptT& log_decay, const OptT& skip, const at::Tensor& cu, at::Tensor loc, at::Tensor dec,
+                        const OptT& trans);
+void memory_combine(at::Tensor S, const at::Tensor& slots, const at::Tensor& start, const at::Tensor& base, const at::Tensor& loc, const at::Tensor& dec,
+                    const OptT& trans, at::Tensor init);
+std::tuple<at::Tensor, at::Tensor> embed_f32(const at::Tensor& ids, const at::Tensor& table);
+at::Tensor norm_add_f32_(at::Tensor x, const at::Tensor& y1, double s1, const OptT& y2, double s2, const at::Tensor& w, double mult, double eps,
+                         bool one_plus, bool out_bf16);
+at::Tensor gate_groupnorm(const at::Tensor& o, const at::Tensor& z, const at::Tensor& w, int64_t groups, double eps, bool out_bf16);
+at::Tensor rotary_f32(const at::Tensor& z, int64_t nq, int64_t nk, int64_t dk, const at::Tensor& pos, const at::Tensor& freq, int64_t rot, bool interleaved,
+                      double amp, double kscale);
 }  // namespace llmctl_hybrid
 
 TORCH_LIBRARY(llmctl_hybrid, m) {
@@ -96,7 +118,7 @@ TORCH_LIBRARY(llmctl_hybrid, m) {
   m.def("add_layernorm_f32_(Tensor(a!) x, Tensor a, Tensor? b, Tensor w, Tensor bias, float eps, bool out_bf16) -> Tensor");
   m.def("rmsnorm_cols(Tensor x, Tensor w, float eps, int n, bool out_bf16) -> Tensor");
   m.def("sigmoid_gate_mul(Tensor o, Tensor g) -> Tensor");
-  m.def("headnorm_gate(Tensor o, Tensor w, Tensor g, float eps, bool out_bf16, bool silu=False) -> Tensor");
+  m.def("headnorm_gate(Tensor o, Tensor? w, Tensor g, float eps, bool out_bf16, bool silu=False) -> Tensor");
   m.def("latent_kv_write(Tensor dkv, Tensor norm_w, float eps, Tensor pos, Tensor inv_freq, int rot_dims, Tensor(a!) cache, Tensor slots, bool interleaved=False, float amp=1.0) -> ()");
   m.def("latent_q_assemble(Tensor q_lat, Tensor q, Tensor pos, Tensor inv_freq, int rot_dims, int dn, bool interleaved=False, float amp=1.0) -> Tensor");
   m.def("latent_attn_prefill(Tensor qa, Tensor cache, Tensor bt, Tensor cu, Tensor ctx, int window, Tensor? sink, float scale, int rk, int max_q, bool mfma=True, int groups=1, int koff=0, int chunk=1073741824, Tensor? hscale=None, Tensor? ofreq=None, Tensor? sig_bias=None, Tensor? dist_a=None, Tensor? dist_b=None, float softcap=0.0, int keep_first=0) -> Tensor");
@@ -120,7 +142,7 @@ TORCH_LIBRARY(llmctl_hybrid, m) {
   m.def("gated_norm_add_norm_f32_(Tensor(a!) x, Tensor y, Tensor r, Tensor w_post, Tensor? w_next, float eps, bool out_bf16) -> Tensor");
   m.def("embed_rmsnorm_f32(Tensor ids, Tensor pos, Tensor table, Tensor pos_table, Tensor w, float eps, bool out_bf16) -> (Tensor, Tensor)");
   m.def("act_any(Tensor x, int kind, Tensor? scale=None) -> Tensor");
-  m.def("qk_fullnorm_prep(Tensor z, int H, int G, int dk, int dv, Tensor q_norm, Tensor k_norm, float eps, Tensor pos, float temp_coef, int temp_every, Tensor(a!) cache, Tensor slots) -> Tensor");
+  m.def("qk_fullnorm_prep(Tensor z, int H, int G, int dk, int dv, Tensor q_norm, Tensor k_norm, float eps, Tensor pos, float temp_coef, int temp_every, Tensor(a!) cache, Tensor slots, Tensor? freq=None, int rot=0, bool interleaved=False, float amp=1.0) -> Tensor");
   m.def("gla_scan(Tensor q, Tensor k, Tensor v, Tensor z, Tensor z_bias, float tau, float qscale, Tensor(a!) S, Tensor slots, Tensor cu, Tensor start, Tensor(b!)? logd=None, bool write_out=True, bool write_state=True) -> Tensor");
   m.def("gla_chunk_combine(Tensor(a!) S, Tensor slots, Tensor start, Tensor base, Tensor loc, Tensor logd, Tensor(b!) init) -> ()");
   m.def("glu_act(Tensor gu, int kind, Tensor? scale=None) -> Tensor");
@@ -130,6 +152,15 @@ TORCH_LIBRARY(llmctl_hybrid, m) {
   m.def("mingru_scan(Tensor z, Tensor z_bias, Tensor x_bias, Tensor(a!) S, Tensor slots, Tensor cu, Tensor start, int portions, int max_q, int chunk) -> Tensor");
   m.def("kv_rows_write(Tensor k, Tensor v, Tensor(a!) cache, Tensor slots, int groups) -> ()");
   m.def("diff_attn(Tensor q, Tensor cache, Tensor bt, Tensor? cu, Tensor ctx, int heads, int groups, int dk, int dv, int window, float scale, Tensor lam, float post, float eps, int max_q, int max_ctx, bool mfma, Tensor(a!) out) -> ()");
+  m.def("conv_silu_unit(Tensor u, Tensor w, Tensor? bias, Tensor(a!) state, Tensor seq_of, Tensor cu, Tensor start, Tensor sslot, int nq, int nk, int dk, float qscale, float eps, int max_len=0) -> (Tensor, Tensor)");
+  m.def("memory_decode(Tensor q, Tensor k, Tensor v, int kind, Tensor? ga, Tensor? gb, Tensor? a_log, Tensor? dt_bias, Tensor? log_decay, Tensor? skip, Tensor(a!) S, Tensor slots, Tensor start, Tensor(b!) out, int row0) -> ()");
+  m.def("memory_chunks(Tensor q, Tensor k, Tensor v, int kind, Tensor? ga, Tensor? gb, Tensor? a_log, Tensor? dt_bias, Tensor? log_decay, Tensor? skip, Tensor(a!) S, Tensor? slots, Tensor cu, Tensor? start, Tensor? init, Tensor(b!) out, int rows) -> ()");
+  m.def("memory_chunk_local(Tensor q, Tensor k, Tensor v, int kind, Tensor? ga, Tensor? gb, Tensor? a_log, Tensor? dt_bias, Tensor? log_decay, Tensor? skip, Tensor cu, Tensor(a!) loc, Tensor(b!) dec, Tensor(c!)? trans) -> ()");
+  m.def("memory_combine(Tensor(a!) S, Tensor slots, Tensor start, Tensor base, Tensor loc, Tensor dec, Tensor? trans, Tensor(b!) init) -> ()");
+  m.def("embed_f32(Tensor ids, Tensor table) -> (Tensor, Tensor)");
+  m.def("norm_add_f32_(Tensor(a!) x, Tensor y1, float s1, Tensor? y2, float s2, Tensor w, float mult, float eps, bool one_plus, bool out_bf16) -> Tensor");
+  m.def("gate_groupnorm(Tensor o, Tensor z, Tensor w, int groups, float eps, bool out_bf16) -> Tensor");
+  m.def("rotary_f32(Tensor z, int nq, int nk, int dk, Tensor pos, Tensor freq, int rot, bool interleaved, float amp, float kscale) -> Tensor");
 }
 
 TORCH_LIBRARY_IMPL(llmctl_hybrid, CUDA, m) {
@@ -172,4 +203,13 @@ TORCH_LIBRARY_IMPL(llmctl_hybrid, CUDA, m) {
   m.impl("mingru_scan", &llmctl_hybrid::mingru_scan);
   m.impl("kv_rows_write", &llmctl_hybrid::kv_rows_write);
   m.impl("diff_attn", &llmctl_hybrid::diff_attn);
+  m.impl("conv_silu_unit", &llmctl_hybrid::conv_silu_unit);
+  m.impl("memory_decode", &llmctl_hybrid::memory_decode);
+  m.impl("memory_chunks", &llmctl_hybrid::memory_chunks);
+  m.impl("memory_chunk_local", &llmctl_hybrid::memory_chunk_local);
+  m.impl("memory_combine", &llmctl_hybrid::memory_combine);
+  m.impl("embed_f32", &llmctl_hybrid::embed_f32);
+  m.impl("norm_add_f32_", &llmctl_hybrid::norm_add_f32_);
+  m.impl("gate_groupnorm", &llmctl_hybrid::gate_groupnorm);
+  m.impl("rotary_f32", &llmctl_hybrid::rotary_f32);
 }

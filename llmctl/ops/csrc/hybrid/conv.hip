@@ -12,6 +12,9 @@
 //                             for portions shorter than taps - 1, the slot's old content
 //   causal_conv_short_kernel  steps whose portions are all short (decode rows): one thread per (sequence,
 //                             channel) walks the portion's tokens and then writes the slot, in one launch
+//   conv_silu_unit_kernel     silu(convolution + bias) for the inputs of a recurrence, the first groups of channels as unit
+//                             vectors in fp32: a group's lanes walk a few tokens with the last inputs in registers;
+//                             steps of short portions write the slots in the same launch
 #include "hybrid_common.h"
 
 namespace llmctl_hybrid {
@@ -180,6 +183,259 @@ at::Tensor causal_conv(const at::Tensor& u, const at::Tensor& w, at::Tensor stat
           (int)C, (int)taps);
   });
   return y;
+}
+
+namespace {
+struct ConvUnitArgs {
+  const void* u;
+  int64_t u_st;
+  const float* w;     // [taps, C]
+  const float* bias;  // nullptr or [C]
+  float* state;       // [slots, taps - 1, C]
+  const int* seq_of;
+  const int* cu;
+  const int* start;
+  const int* sslot;
+  float* qk;  // [T, ng, dk]
+  void* y;    // [T, C - ng * dk]
+  int T, C, taps, ng, nq, dk, lg, tok, whole;  // lg lanes per unit; tok tokens per walk, or (whole) a sequence per walk
+  float qscale, eps;
+};
+
+// A unit is a group of dk channels, or a span of lg * VEC * NI of the other channels.  TAPS == 0: any number of taps.
+template <typename T, int VEC, int NI, int TAPS>
+__global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
+  constexpr int NH = TAPS > 1 ? TAPS - 1 : 1;
+  const int lane = threadIdx.x % a.lg;
+  const int unit = ((int)blockIdx.y * 256 + (int)threadIdx.x) / a.lg;
+  const int taps = TAPS > 0 ? TAPS : a.taps;
+  const int span = a.lg * VEC * NI, gw = a.ng * a.dk;
+  const bool grp = unit < a.ng;
+  const int base = grp ? unit * a.dk : gw + (unit - a.ng) * span;
+  const int lim = grp ? base + a.dk : min(base + span, a.C);
+  if (base >= a.C) return;  // (the unit's lanes leave together)
+  int t_lo, t_hi;
+  if (a.whole) {
+    t_lo = a.cu[blockIdx.x], t_hi = a.cu[blockIdx.x + 1];
+    if (t_lo >= t_hi) return;
+  } else {
+    t_lo = (int)blockIdx.x * a.tok, t_hi = min(t_lo + a.tok, a.T);
+  }
+  const T* u = reinterpret_cast<const T*>(a.u);
+  int ch[NI];
+  bool ok[NI];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    ch[i] = base + (i * a.lg + lane) * VEC;
+    ok[i] = ch[i] < lim;  // VEC divides the group and the row
+    if (!ok[i]) ch[i] = base;
+  }
+  auto load_row = [&](const T* p, float* v) {
+    if constexpr (VEC == 4 && sizeof(T) == 4) {
+      Vec16<float>::load(reinterpret_cast<const float*>(p), v);
+    } else if constexpr (VEC == 4) {
+      const uint2 x = *reinterpret_cast<const uint2*>(p);
+      v[0] = __uint_as_float(x.x << 16), v[1] = __uint_as_float(x.x & 0xffff0000u);
+      v[2] = __uint_as_float(x.y << 16), v[3] = __uint_as_float(x.y & 0xffff0000u);
+    } else {
+      v[0] = ldf(p);
+    }
+  };
+  auto load_f = [&](const float* p, float* v) {
+    if constexpr (VEC == 4) Vec16<float>::load(p, v);
+    else v[0] = p[0];
+  };
+  // the input ``k`` positions before token t of the sequence that begins at row s0, position p0
+  auto past = [&](int t, int k, int s0, int p0, const float* st, int i, float* v) {
+    const int j = t - s0 - k;
+    if (j >= 0) {
+      load_row(u + (int64_t)(t - k) * a.u_st + ch[i], v);
+    } else if (p0 + j >= 0) {
+      load_f(st + (int64_t)(taps - 1 + j) * a.C + ch[i], v);
+    } else {
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) v[c] = 0.f;
+    }
+  };
+  float wk[TAPS > 0 ? TAPS : 1][NI][VEC], bs[NI][VEC];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+#pragma unroll
+    for (int c = 0; c < VEC; ++c) bs[i][c] = 0.f;
+    if (a.bias != nullptr) load_f(a.bias + ch[i], bs[i]);
+    if constexpr (TAPS > 0) {
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) load_f(a.w + (int64_t)k * a.C + ch[i], wk[k][i]);
+    }
+  }
+  float hist[NH][NI][VEC];  // hist[k]: the input k + 1 positions before the current token
+  int s = a.whole ? (int)blockIdx.x : a.seq_of[t_lo];
+  int s0 = a.cu[s], s1 = a.cu[s + 1], p0 = a.start[s];
+  float* st = a.state + (int64_t)a.sslot[s] * (taps - 1) * a.C;
+  for (int t = t_lo; t < t_hi; ++t) {
+    bool reload = t == t_lo;
+    if (t >= s1) {
+      s = a.seq_of[t];
+      s0 = a.cu[s], s1 = a.cu[s + 1], p0 = a.start[s];
+      st = a.state + (int64_t)a.sslot[s] * (taps - 1) * a.C;
+      reload = true;
+    }
+    if constexpr (TAPS > 1) {
+      if (reload) {
+#pragma unroll
+        for (int k = 0; k < TAPS - 1; ++k)
+#pragma unroll
+          for (int i = 0; i < NI; ++i) past(t, k + 1, s0, p0, st, i, hist[k][i]);
+      }
+    }
+    float x[NI][VEC], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      float cur[VEC];
+      load_row(u + (int64_t)t * a.u_st + ch[i], cur);
+      if constexpr (TAPS > 0) {
+#pragma unroll
+        for (int c = 0; c < VEC; ++c) {
+          float acc = bs[i][c] + wk[TAPS - 1][i][c] * cur[c];
+#pragma unroll
+          for (int k = 0; k < TAPS - 1; ++k) acc += wk[TAPS - 2 - k][i][c] * hist[k][i][c];
+          x[i][c] = acc;
+        }
+#pragma unroll
+        for (int k = TAPS - 2; k > 0; --k)
+#pragma unroll
+          for (int c = 0; c < VEC; ++c) hist[k][i][c] = hist[k - 1][i][c];
+        if constexpr (TAPS > 1) {
+#pragma unroll
+          for (int c = 0; c < VEC; ++c) hist[0][i][c] = cur[c];
+        }
+      } else {
+        float w1[VEC], v[VEC];
+        load_f(a.w + (int64_t)(taps - 1) * a.C + ch[i], w1);
+#pragma unroll
+        for (int c = 0; c < VEC; ++c) x[i][c] = bs[i][c] + w1[c] * cur[c];
+        for (int k = 1; k < taps; ++k) {
+          past(t, k, s0, p0, st, i, v);
+          load_f(a.w + (int64_t)(taps - 1 - k) * a.C + ch[i], w1);
+#pragma unroll
+          for (int c = 0; c < VEC; ++c) x[i][c] += w1[c] * v[c];
+        }
+      }
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) {
+        x[i][c] = x[i][c] / (1.0f + expf(-x[i][c]));
+        if (ok[i]) ss += x[i][c] * x[i][c];
+      }
+    }
+    if (grp) {
+      for (int o = a.lg >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+      const float f = (unit < a.nq ? a.qscale : 1.0f) / sqrtf(ss + a.eps);
+      float* o = a.qk + ((int64_t)t * a.ng + unit) * a.dk - base;
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+#pragma unroll
+        for (int c = 0; c < VEC; ++c) x[i][c] *= f;
+        if (ok[i]) {
+          if constexpr (VEC == 4) Vec16<float>::store(o + ch[i], x[i]);
+          else o[ch[i]] = x[i][0];
+        }
+      }
+    } else {
+      T* o = reinterpret_cast<T*>(a.y) + (int64_t)t * (a.C - gw) - gw;
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        if (!ok[i]) continue;
+        if constexpr (VEC == 4 && sizeof(T) == 4) {
+          Vec16<float>::store(reinterpret_cast<float*>(o) + ch[i], x[i]);
+        } else if constexpr (VEC == 4) {
+          unsigned w[2];
+#pragma unroll
+          for (int c = 0; c < 2; ++c)
+            w[c] = (unsigned)__bfloat16_as_ushort(__float2bfloat16(x[i][2 * c])) | ((unsigned)__bfloat16_as_ushort(__float2bfloat16(x[i][2 * c + 1])) << 16);
+          *reinterpret_cast<uint2*>(o + ch[i]) = make_uint2(w[0], w[1]);
+        } else {
+          stf(o + ch[i], x[i][0]);
+        }
+      }
+    }
+  }
+  if (a.whole) {  // the slot's new content; entry j is the input taps - 1 - j positions before the portion's end
+    for (int j = 0; j < taps - 1; ++j) {
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        float v[VEC];
+        past(t_hi, taps - 1 - j, s0, p0, st, i, v);  // (ascending j reads entries that are not yet rewritten)
+        if (ok[i]) {
+#pragma unroll
+          for (int c = 0; c < VEC; ++c) st[(int64_t)j * a.C + ch[i] + c] = v[c];
+        }
+      }
+    }
+  }
+}
+}  // namespace
+
+// max_len: the longest portion of the step
+std::tuple<at::Tensor, at::Tensor> conv_silu_unit(const at::Tensor& u, const at::Tensor& w, const c10::optional<at::Tensor>& bias, at::Tensor state,
+                                                  const at::Tensor& seq_of, const at::Tensor& cu, const at::Tensor& start, const at::Tensor& sslot,
+                                                  int64_t nq, int64_t nk, int64_t dk, double qscale, double eps, int64_t max_len) {
+  check_rows(u, "u");
+  const int64_t T = u.size(0), C = u.size(1), ng = nq + nk;
+  auto f32c = [](const at::Tensor& t) { return t.is_cuda() && t.is_contiguous() && t.scalar_type() == at::kFloat; };
+  HYB_CHECK(f32c(w) && w.dim() == 2 && w.size(1) == C && w.size(0) >= 1 && w.size(0) <= CONV_MAX_TAPS, "w: contiguous fp32 [taps, C], 1 .. 16 taps");
+  const int64_t taps = w.size(0);
+  HYB_CHECK(!bias.has_value() || (f32c(*bias) && bias->numel() == C), "bias: fp32 [C]");
+  HYB_CHECK(f32c(state) && state.dim() == 3 && state.size(1) == taps - 1 && state.size(2) == C, "state: contiguous fp32 [slots, taps - 1, C]");
+  auto i32 = [](const at::Tensor& t) { return t.is_cuda() && t.is_contiguous() && t.scalar_type() == at::kInt; };
+  HYB_CHECK(i32(seq_of) && i32(cu) && i32(start) && i32(sslot), "seq_of, cu, start, slots: contiguous int32 GPU tensors");
+  const int64_t ns = start.numel();
+  HYB_CHECK(seq_of.numel() == T && cu.numel() == ns + 1 && sslot.numel() == ns, "seq_of [T], cu [n + 1], start [n], slots [n]");
+  HYB_CHECK(nq >= 0 && nk >= 0 && (ng == 0 || (dk >= 1 && dk <= 256)) && ng * dk <= C, "groups of 1 .. 256 channels inside the row");
+  if (ng == 0) dk = 0;
+  c10::DeviceGuard guard(u.device());
+  at::Tensor qk = at::empty({T, ng, dk}, u.options().dtype(at::kFloat));
+  at::Tensor y = at::empty({T, C - ng * dk}, u.options());
+  if (T == 0 || C == 0) return {qk, y};
+  const bool v4 = dk % 4 == 0 && C % 4 == 0 && u.stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(u.data_ptr()) % (4 * u.element_size()) == 0;
+  const int64_t vec = v4 ? 4 : 1;
+  int lg = 64;
+  if (ng > 0)
+    for (lg = 1; lg < 64 && lg * vec < dk;) lg *= 2;
+  const int ni = ng > 0 ? (int)((dk + lg * vec - 1) / (lg * vec)) : 1;  // 1, or up to 4 in the scalar form
+  ConvUnitArgs a;
+  a.u = u.data_ptr(), a.u_st = u.stride(0), a.w = w.data_ptr<float>(), a.bias = bias.has_value() ? bias->data_ptr<float>() : nullptr;
+  a.state = state.data_ptr<float>(), a.seq_of = seq_of.data_ptr<int>(), a.cu = cu.data_ptr<int>(), a.start = start.data_ptr<int>(), a.sslot = sslot.data_ptr<int>();
+  a.qk = qk.data_ptr<float>(), a.y = y.data_ptr();
+  a.T = (int)T, a.C = (int)C, a.taps = (int)taps, a.ng = (int)ng, a.nq = (int)nq, a.dk = (int)dk, a.lg = lg;
+  a.whole = max_len >= 1 && max_len <= CONV_SHORT ? 1 : 0;
+  a.qscale = (float)qscale, a.eps = (float)eps;
+  const int NIv = ni > 1 ? 4 : 1;
+  const int64_t span = (int64_t)lg * vec * NIv, units = ng + (C - ng * dk + span - 1) / span;
+  const int64_t by = (units * lg + 255) / 256;
+  a.tok = 1;  // tokens per walk: as many as leave the chip a few thousand workgroups
+  while (a.tok < 16 && T * by / (2 * a.tok) >= 2048) a.tok *= 2;
+  HYB_CHECK(by <= 65535, "too many channels for one launch");
+  const dim3 grid((unsigned)(a.whole ? ns : (T + a.tok - 1) / a.tok), (unsigned)by);
+  dispatch_act(u, [&](auto* tag) {
+    using Tt = std::remove_pointer_t<decltype(tag)>;
+    auto go = [&](auto kern) { kern<<<grid, 256, 0, cur_stream()>>>(a); };
+    auto taps_of = [&](auto vc, auto nc) {
+      constexpr int V = decltype(vc)::value, N = decltype(nc)::value;
+      switch (taps) {
+        case 2: go(conv_silu_unit_kernel<Tt, V, N, 2>); break;
+        case 3: go(conv_silu_unit_kernel<Tt, V, N, 3>); break;
+        case 4: go(conv_silu_unit_kernel<Tt, V, N, 4>); break;
+        default: go(conv_silu_unit_kernel<Tt, V, N, 0>); break;
+      }
+    };
+    if (v4) taps_of(std::integral_constant<int, 4>(), std::integral_constant<int, 1>());
+    else if (NIv == 1) taps_of(std::integral_constant<int, 1>(), std::integral_constant<int, 1>());
+    else taps_of(std::integral_constant<int, 1>(), std::integral_constant<int, 4>());
+    if (!a.whole && taps > 1)
+      causal_conv_state_kernel<Tt><<<dim3((unsigned)ns, (unsigned)((C + 255) / 256)), 256, 0, cur_stream()>>>(
+          (const Tt*)u.data_ptr(), u.stride(0), state.data_ptr<float>(), cu.data_ptr<int>(), start.data_ptr<int>(), sslot.data_ptr<int>(), (int)C, (int)taps);
+  });
+  return {qk, y};
 }
 
 }  // namespace llmctl_hybrid

@@ -3,6 +3,7 @@
 //   gated_norm_add_norm_f32_  g = y sigmoid(r); x += g / rms(g) * w_post; h = x / rms(x) * w_next, one pass per row
 //   embed_rmsnorm_f32         x = table[id] + pos_table[position] as the fp32 stream, and its first RMS norm
 //   act_any                   relu(x)^2 or the exact (erf) GELU on a column range of a wider row
+//   qk_fullnorm_prep          queries and keys normed as whole rows, turned by their position, keys and values to the cache
 //   glu_act                   act(gate) * up of rows [gate | up] (silu or the tanh GELU), times an optional factor per row
 // All arithmetic fp32; y, r, h in the activation dtype or fp32.
 #include "hybrid_common.h"
@@ -147,41 +148,116 @@ __global__ __launch_bounds__(256) void glu_act_kernel(const T* __restrict__ gu, 
   else Vec16<T>::store(y + r * F + c, g);
 }
 
+template <typename T, int N>
+__device__ __forceinline__ void ld_piece(const T* p, float* v) {  // N neighbouring elements (N == 4: one access)
+  if constexpr (N == 1) {
+    v[0] = ldf(p);
+  } else if constexpr (sizeof(T) == 4) {
+    Vec16<float>::load(reinterpret_cast<const float*>(p), v);
+  } else {
+    const uint2 x = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(x.x << 16), v[1] = __uint_as_float(x.x & 0xffff0000u);
+    v[2] = __uint_as_float(x.y << 16), v[3] = __uint_as_float(x.y & 0xffff0000u);
+  }
+}
+template <typename T, int N>
+__device__ __forceinline__ void st_piece(T* p, const float* v) {
+  if constexpr (N == 1) {
+    stf(p, v[0]);
+  } else if constexpr (sizeof(T) == 4) {
+    Vec16<float>::store(reinterpret_cast<float*>(p), v);
+  } else {
+    unsigned w[2];
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+      w[c] = (unsigned)__bfloat16_as_ushort(__float2bfloat16(v[2 * c])) | ((unsigned)__bfloat16_as_ushort(__float2bfloat16(v[2 * c + 1])) << 16);
+    *reinterpret_cast<uint2*>(p) = make_uint2(w[0], w[1]);
+  }
+}
+
 // z [T, >= H*dk + G*dk + G*dv] = [q | k | v | ...]: unit RMS over all of q and over all of k, times the weights;
-// q times the position's temperature; [v | k] per kv group to the token's cache row.  One block per token.
-template <typename T>
+// q times the position's temperature; rotary of q and k on the first rot entries of every head (halves, or neighbours
+// when inter); [v | k] per kv group to the token's cache row.  One block per token; pieces of N neighbouring elements.
+template <typename T, int N>
 __global__ __launch_bounds__(NT) void qk_fullnorm_prep_kernel(const T* __restrict__ z, int64_t z_st, const float* __restrict__ wq,
                                                               const float* __restrict__ wk, const int* __restrict__ pos, T* __restrict__ q,
                                                               T* __restrict__ cache, const int64_t* __restrict__ slots, int H, int G, int dk,
-                                                              int dv, float eps, float coef, int every) {
-  __shared__ float red[NW];
+                                                              int dv, float eps, float coef, int every, const float* __restrict__ freq, int rot,
+                                                              int inter, float amp) {
+  extern __shared__ float cs[];  // [rot / 2] cos, then [rot / 2] sin
+  __shared__ float red[2 * NW];
   const int64_t t = blockIdx.x;
   const T* zr = z + t * z_st;
-  const int nq = H * dk, nk = G * dk, nv = G * dv;
+  const int nq = H * dk, nk = G * dk, nv = G * dv, half = rot / 2;
+  const float p = (float)pos[t];
+  for (int i = threadIdx.x; i < half; i += NT) {
+    float s, c;
+    sincosf(p * freq[i], &s, &c);
+    cs[i] = c * amp;
+    cs[half + i] = s * amp;
+  }
   float sq = 0.f, sk = 0.f;
-  for (int c = threadIdx.x; c < nq; c += NT) {
-    const float v = ldf(zr + c);
-    sq += v * v;
+  for (int c = threadIdx.x * N; c < nq + nk; c += NT * N) {  // (N divides nq)
+    float v[N], a = 0.f;
+    ld_piece<T, N>(zr + c, v);
+#pragma unroll
+    for (int i = 0; i < N; ++i) a += v[i] * v[i];
+    if (c < nq) sq += a;
+    else sk += a;
   }
-  for (int c = threadIdx.x; c < nk; c += NT) {
-    const float v = ldf(zr + nq + c);
-    sk += v * v;
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((threadIdx.x & 63) == 0) {
+    red[threadIdx.x >> 6] = sq;
+    red[NW + (threadIdx.x >> 6)] = sk;
   }
-  const float rq = 1.0f / sqrtf(block_sum<NW>(sq, red) / (float)nq + eps);
-  const float rk = 1.0f / sqrtf(block_sum<NW>(sk, red) / (float)nk + eps);
+  __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NW; ++i) sq += red[i], sk += red[NW + i];
   float temp = 1.0f;
   if (coef != 0.f) temp = 1.0f + coef * logf((float)((pos[t] + 1) / every) + 1.0f);
-  for (int c = threadIdx.x; c < nq; c += NT) stf(q + t * nq + c, ldf(zr + c) * rq * wq[c] * temp);
+  const float rq = temp / sqrtf(sq / (float)nq + eps), rk = 1.0f / sqrtf(sk / (float)nk + eps);
   const int64_t slot = slots[t];
-  if (slot < 0) return;
   T* row = cache + slot * (int64_t)(nk + nv);
-  for (int c = threadIdx.x; c < nk; c += NT) {
-    const int g = c / dk, d = c - g * dk;
-    stf(row + g * (dv + dk) + dv + d, ldf(zr + nq + c) * rk * wk[c]);
+  auto normed = [&](int c, float* v) {  // N entries of the row [q | k] from column c on, normed
+    float w[N];
+    ld_piece<T, N>(zr + c, v);
+    ld_piece<float, N>(c < nq ? wq + c : wk + (c - nq), w);
+    const float f = c < nq ? rq : rk;
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] *= f * w[i];
+  };
+  for (int c = threadIdx.x * N; c < nq + nk; c += NT * N) {
+    const int hd = c / dk, d = c - hd * dk;
+    float v[N], m[N];
+    normed(c, v);
+    if (d < rot) {
+      if (inter) {
+        if constexpr (N == 1) normed(c - d + (d ^ 1), m);
+        else m[0] = v[1], m[1] = v[0], m[2] = v[3], m[3] = v[2];
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+          const int di = d + i;
+          if (di < rot) v[i] = v[i] * cs[di >> 1] + ((di & 1) ? m[i] : -m[i]) * cs[half + (di >> 1)];
+        }
+      } else {  // N == 4: half is a multiple of 4, so a piece lies on one side
+        const bool first = d < half;
+        normed(c + (first ? half : -half), m);
+        const int i0 = first ? d : d - half;
+#pragma unroll
+        for (int i = 0; i < N; ++i) v[i] = v[i] * cs[i0 + i] + (first ? -m[i] : m[i]) * cs[half + i0 + i];
+      }
+    }
+    if (c < nq) st_piece<T, N>(q + t * nq + c, v);
+    else if (slot >= 0) st_piece<T, N>(row + (hd - H) * (dv + dk) + dv + d, v);
   }
-  for (int c = threadIdx.x; c < nv; c += NT) {
+  if (slot < 0) return;
+  for (int c = threadIdx.x * N; c < nv; c += NT * N) {
     const int g = c / dv, d = c - g * dv;
-    row[g * (dv + dk) + d] = zr[nq + nk + c];
+    float v[N];
+    ld_piece<T, N>(zr + nq + nk + c, v);
+    st_piece<T, N>(row + g * (dv + dk) + d, v);
   }
 }
 
@@ -298,7 +374,8 @@ at::Tensor glu_act(const at::Tensor& gu, int64_t kind, const c10::optional<at::T
 }
 
 at::Tensor qk_fullnorm_prep(const at::Tensor& z, int64_t H, int64_t G, int64_t dk, int64_t dv, const at::Tensor& q_norm, const at::Tensor& k_norm,
-                            double eps, const at::Tensor& pos, double temp_coef, int64_t temp_every, at::Tensor cache, const at::Tensor& slots) {
+                            double eps, const at::Tensor& pos, double temp_coef, int64_t temp_every, at::Tensor cache, const at::Tensor& slots,
+                            const c10::optional<at::Tensor>& freq, int64_t rot, bool interleaved, double amp) {
   check_rows(z, "z");
   const int64_t T = z.size(0);
   HYB_CHECK(H >= 1 && G >= 1 && H % G == 0 && dk >= 1 && dv >= 1 && z.size(1) >= (H + G) * dk + G * dv, "z: [T, >= H*dk + G*dk + G*dv]");
@@ -309,15 +386,24 @@ at::Tensor qk_fullnorm_prep(const at::Tensor& z, int64_t H, int64_t G, int64_t d
                 slots.scalar_type() == at::kLong && slots.numel() == T,
             "pos int32 [T], slots int64 [T]");
   HYB_CHECK(temp_every >= 1, "temperature period >= 1");
+  HYB_CHECK(rot >= 0 && rot % 2 == 0 && rot <= dk && rot <= 8192 && (rot == 0 || (freq.has_value() && f32w(*freq, rot / 2))),
+            "rotary: even dims <= dk, fp32 frequencies [dims / 2]");
   c10::DeviceGuard guard(z.device());
   at::Tensor q = at::empty({T, H, dk}, z.options());
   if (T == 0) return q;
   dispatch_act(z, [&](auto* tag) {
     using Tt = std::remove_pointer_t<decltype(tag)>;
-    qk_fullnorm_prep_kernel<Tt><<<dim3((unsigned)T), NT, 0, cur_stream()>>>((const Tt*)z.data_ptr(), z.stride(0), q_norm.data_ptr<float>(),
-                                                                           k_norm.data_ptr<float>(), pos.data_ptr<int>(), (Tt*)q.data_ptr(),
-                                                                           (Tt*)cache.data_ptr(), slots.data_ptr<int64_t>(), (int)H, (int)G, (int)dk,
-                                                                           (int)dv, (float)eps, (float)temp_coef, (int)temp_every);
+    auto a16 = [](const at::Tensor& t) { return reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0; };
+    const bool v4 = dk % 4 == 0 && dv % 4 == 0 && (interleaved || (rot / 2) % 4 == 0) && z.stride(0) % 4 == 0 &&
+                    reinterpret_cast<uintptr_t>(z.data_ptr()) % (4 * sizeof(Tt)) == 0 && a16(q_norm) && a16(k_norm) && a16(cache);
+    auto go = [&](auto kern) {
+      kern<<<dim3((unsigned)T), NT, (size_t)rot * sizeof(float), cur_stream()>>>(
+          (const Tt*)z.data_ptr(), z.stride(0), q_norm.data_ptr<float>(), k_norm.data_ptr<float>(), pos.data_ptr<int>(), (Tt*)q.data_ptr(),
+          (Tt*)cache.data_ptr(), slots.data_ptr<int64_t>(), (int)H, (int)G, (int)dk, (int)dv, (float)eps, (float)temp_coef, (int)temp_every,
+          rot > 0 ? freq->data_ptr<float>() : nullptr, (int)rot, interleaved ? 1 : 0, (float)amp);
+    };
+    if (v4) go(qk_fullnorm_prep_kernel<Tt, 4>);
+    else go(qk_fullnorm_prep_kernel<Tt, 1>);
   });
   return q;
 }

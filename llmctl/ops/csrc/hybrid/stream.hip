@@ -154,7 +154,7 @@ __global__ void gate_mul_kernel(const TO* __restrict__ o, const TG* __restrict__
   stf(y + i, ldf(o + i) * (1.0f / (1.0f + expf(-gv))));
 }
 
-// o [T, H, dv] fp32 -> y [T, H*dv]: o / rms(o over dv) * w * sigmoid(g) (silu: * g sigmoid(g)); one wave per (token, head).
+// o [T, H, dv] fp32 -> y [T, H*dv]: o / rms(o over dv) * w (if given) * sigmoid(g) (silu: * g sigmoid(g)); one wave per (token, head).
 template <typename T>
 __global__ __launch_bounds__(NT) void headnorm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w,
                                                            const T* __restrict__ g, int64_t g_stride, T* __restrict__ y,
@@ -171,7 +171,7 @@ __global__ __launch_bounds__(NT) void headnorm_gate_kernel(const float* __restri
   for (int c = lane; c < dv; c += 64) {
     const float gv = ldf(g + t * g_stride + hd * dv + c);
     const float gate = 1.0f / (1.0f + expf(-gv));
-    stf(y + p * dv + c, op[c] * rstd * w[hd * dv + c] * (silu ? gv * gate : gate));
+    stf(y + p * dv + c, op[c] * rstd * (w != nullptr ? w[hd * dv + c] : 1.0f) * (silu ? gv * gate : gate));
   }
 }
 
@@ -336,12 +336,12 @@ at::Tensor clamped_glu(const at::Tensor& gu, double limit, double alpha) {
   return y;
 }
 
-at::Tensor headnorm_gate(const at::Tensor& o, const at::Tensor& w, const at::Tensor& g, double eps, bool out_bf16, bool silu) {
+at::Tensor headnorm_gate(const at::Tensor& o, const c10::optional<at::Tensor>& w, const at::Tensor& g, double eps, bool out_bf16, bool silu) {
   HYB_CHECK(o.is_cuda() && o.is_contiguous() && o.dim() == 3 && o.scalar_type() == at::kFloat, "o: contiguous fp32 [T, H, dv]");
   check_rows(g, "g");
   const int64_t T = o.size(0);
   const int H = (int)o.size(1), dv = (int)o.size(2);
-  HYB_CHECK(g.size(0) == T && g.size(1) == (int64_t)H * dv && w.numel() == (int64_t)H * dv && w.scalar_type() == at::kFloat && w.is_contiguous(), "g [T, H*dv], w fp32 [H*dv]");
+  HYB_CHECK(g.size(0) == T && g.size(1) == (int64_t)H * dv && (!w.has_value() || (w->numel() == (int64_t)H * dv && w->scalar_type() == at::kFloat && w->is_contiguous())), "g [T, H*dv], w fp32 [H*dv]");
   HYB_CHECK((g.scalar_type() == at::kBFloat16) == out_bf16, "the output has g's dtype");
   c10::DeviceGuard guard(o.device());
   at::Tensor y = out_like(o, {T, (int64_t)H * dv}, out_bf16);
@@ -350,7 +350,7 @@ at::Tensor headnorm_gate(const at::Tensor& o, const at::Tensor& w, const at::Ten
   dispatch_act(g, [&](auto* tag) {
     using Tt = std::remove_pointer_t<decltype(tag)>;
     headnorm_gate_kernel<Tt><<<dim3((unsigned)((pairs + NW - 1) / NW)), NT, 0, cur_stream()>>>(
-        o.data_ptr<float>(), w.data_ptr<float>(), (const Tt*)g.data_ptr(), g.stride(0), (Tt*)y.data_ptr(), pairs, H, dv, (float)eps, silu ? 1 : 0);
+        o.data_ptr<float>(), w.has_value() ? w->data_ptr<float>() : nullptr, (const Tt*)g.data_ptr(), g.stride(0), (Tt*)y.data_ptr(), pairs, H, dv, (float)eps, silu ? 1 : 0);
   });
   return y;
 }

@@ -232,8 +232,8 @@ def _mlstm_scan_chunked(q, k, v, if_raw, b_i, b_f, cap, qscale, S, n, m, state_s
 
 
 def headnorm_gate(o, w, g, eps: float, out_dtype, silu: bool = False):
-    """Per-head unit-RMS of ``o [T, H, dv]`` (fp32), times ``w [H*dv]``, times ``sigmoid(g)`` (``silu``:
-    times ``g sigmoid(g)``)."""
+    """Per-head unit-RMS of ``o [T, H, dv]`` (fp32), times ``w [H*dv]`` (None: no weight), times ``sigmoid(g)``
+    (``silu``: times ``g sigmoid(g)``)."""
     if use_native(o):
         return native_hybrid().headnorm_gate(o, w, g, eps, out_dtype == torch.bfloat16, silu)
     return ref.headnorm_gate(o, w, g, eps, out_dtype, silu)
@@ -340,14 +340,16 @@ def _gla_scan_chunked(nat, q, k, v, z, z_bias, tau, qscale, S, state_slots, star
 
 
 def qk_fullnorm_prep(z, H: int, G: int, dk: int, dv: int, q_norm, k_norm, eps: float, pos, temp_coef: float,
-                     temp_every: int, cache, slots):
+                     temp_every: int, cache, slots, freq=None, rot_dims: int = 0, interleaved: bool = False, amp: float = 1.0):
     """``z [T, >= H*dk + G*dk + G*dv] = [q | k | v | ...]`` (biases already added): RMS norm over the whole
     of q and over the whole of k before the split into heads (weights fp32 ``[H*dk]``, ``[G*dk]``); the query
-    temperature ``1 + temp_coef ln(floor((p + 1) / temp_every) + 1)`` at position p (``temp_coef`` 0: none);
-    k and v are written to the token's cache row ``[G, dv + dk] = [v | k]`` at ``slots``; returns q ``[T, H, dk]``."""
-    if use_native(z):
-        return native_hybrid().qk_fullnorm_prep(z, H, G, dk, dv, q_norm, k_norm, eps, pos, temp_coef, temp_every, cache, slots)
-    return ref.qk_fullnorm_prep(z, H, G, dk, dv, q_norm, k_norm, eps, pos, temp_coef, temp_every, cache, slots)
+    temperature ``1 + temp_coef ln(floor((p + 1) / temp_every) + 1)`` at position p (``temp_coef`` 0: none); rotary of
+    q and k on the first ``rot_dims`` entries of every head (0: none; pairs are neighbours or halves, ``freq`` fp32
+    ``[rot_dims / 2]``, cos and sin times ``amp``); k and v are written to the token's cache row ``[G, dv + dk] = [v | k]``
+    at ``slots``; returns q ``[T, H, dk]``."""
+    a = (z, H, G, dk, dv, q_norm, k_norm, eps, pos, temp_coef, temp_every, cache, slots, freq if rot_dims else None, rot_dims,
+         interleaved, amp)
+    return native_hybrid().qk_fullnorm_prep(*a) if use_native(z) else ref.qk_fullnorm_prep(*a)
 
 
 def bias_topk_router(logits, bias, top: int, groups: int = 1, keep: int = 1, renorm: bool = True):
@@ -559,3 +561,112 @@ def diff_attention(q, cache, bt, cu, ctx, heads: int, groups: int, dk: int, dv: 
     else:
         ref.diff_attention(q, cache, bt, cu, ctx, heads, groups, dk, dv, window, scale, lam, post, eps, out)
     return out
+
+
+def conv_silu_unit(u, w, bias, state, b, nq: int, nk: int, dk: int, qscale: float, eps: float = 1e-6):
+    """Short causal convolutions over time with silu, ``silu(sum_j w[j] u_(t - taps + 1 + j) + bias)`` per channel of the packed
+    rows ``u [T, C]`` (``w`` fp32, tap-major ``[taps, C]``; ``bias`` fp32 ``[C]`` or None), for the inputs of a recurrence:
+    the first ``nq`` groups of ``dk`` channels, then ``nk`` more, become unit vectors ``x / sqrt(sum x^2 + eps)`` (the first
+    ones times ``qscale``).  ``state`` (fp32 ``[slots, taps - 1, C]``) carries each live sequence's last ``taps - 1`` inputs.
+    Returns (unit vectors fp32 ``[T, nq + nk, dk]`` or None, the other channels ``[T, C - (nq + nk) dk]`` in u's dtype)."""
+    if use_native(u):
+        qk, y = native_hybrid().conv_silu_unit(u, w, bias, state, b.seq_of, b.cu, b.start, b.state, nq, nk, dk, qscale, eps,
+                                               max(b.max_q, 1 if u.shape[0] > b.Tp else 0))
+        return (qk if nq + nk else None), y
+    return ref.conv_silu_unit(u, w, bias, state, b.cu, b.start, b.state, nq, nk, dk, qscale, eps)
+
+
+def rotary_f32(z, nq: int, nk: int, dk: int, pos, freq, rot_dims: int, interleaved: bool, amp: float = 1.0, kscale: float = 1.0):
+    """Rotary of the heads ``z [T, >= (nq + nk) dk]`` (``nq`` query heads, then ``nk`` key heads; pairs are halves, or
+    neighbours when ``interleaved``) for a recurrence: fp32 ``[T, nq + nk, dk]``, keys times ``kscale`` after the turn."""
+    a = (z, nq, nk, dk, pos, freq, rot_dims, interleaved, amp, kscale)
+    return native_hybrid().rotary_f32(*a) if use_native(z) else ref.rotary_f32(*a)
+
+
+MEMORY_CHUNK = 64  # tokens per chunk of a memory scan
+MEMORY_KINDS = {"fixed": 0, "ssm": 1, "delta": 2}
+
+
+def _memory_plan(b, device):
+    """The chunks of a step's prompt portions when one of them is longer than a chunk, else None: (chunk row offsets, first
+    chunk of every portion) on ``device`` and the number of chunks.  It depends on the step only; layers share it."""
+    if "memory_plan" not in b.scratch:
+        plan = None
+        if b.max_q > MEMORY_CHUNK:
+            n = b.p_ctx.shape[0]
+            pcu, base = [0], [0]
+            for lo, hi in zip(b.cu_host[:n], b.cu_host[1:n + 1]):
+                pcu += list(range(lo + MEMORY_CHUNK, hi, MEMORY_CHUNK)) + ([hi] if hi > lo else [])
+                base.append(len(pcu) - 1)
+            both = torch.tensor(pcu + base, dtype=torch.int32).to(device)  # blocking: the host tensor is a temporary
+            plan = (both[:len(pcu)], both[len(pcu):], len(pcu) - 1)
+        b.scratch["memory_plan"] = plan
+    return b.scratch["memory_plan"]
+
+
+def memory_scan(q, k, v, kind: str, S, b, ga=None, gb=None, a_log=None, dt_bias=None, log_decay=None, skip=None):
+    """A matrix memory per head with one decay per head and token, over the step's tokens: ``S <- g S``, ``S <- S + k u^T``,
+    ``o = S^T q`` with ``u = beta v``, or ``u = beta (v - S^T k)`` (what the decayed memory gives for k is taken off first).
+
+    ``kind`` says where g and beta come from (fp32 here): ``fixed``: ``g = exp(log_decay_h)``, beta = 1; ``ssm``: ``beta = dt =
+    softplus(ga + dt_bias)``, ``g = exp(-exp(a_log) dt)``; ``delta``: g likewise, ``beta = sigmoid(gb)`` and the subtracting
+    form of u.  ``q, k [T, KH, dk]`` (one dtype; head h of H reads h // (H / KH)), ``v [T, H, dv]`` (row-strided views
+    allowed), ``ga, gb [T, H]`` in v's dtype, ``a_log, dt_bias, log_decay, skip`` fp32 ``[H]``; ``skip``: o gains ``skip_h v``.
+    Returns fp32 ``[T, H, dv]`` and updates the state pool ``S`` (fp32 ``[slots, H, dk, dv]``) in place at ``b.state`` (a
+    sequence that starts at position 0 begins from zeros).
+
+    Decode rows run one after the other in memory (a read and a write of S); prompt portions run in chunks of
+    :data:`MEMORY_CHUNK` tokens whose products go to the fp32 matrix cores.  A portion of several chunks takes three
+    passes: every chunk's own contribution (delta: and its transition product) at once, the memories at the
+    chunks' first tokens in order, every chunk's outputs at once."""
+    if not use_native(v):
+        return ref.memory_scan(q, k, v, kind, ga, gb, a_log, dt_bias, log_decay, skip, S, b.state, b.cu, b.start)
+    nat = native_hybrid()
+    T, H, dv = v.shape
+    dk = q.shape[2]
+    out = torch.empty(T, H, dv, device=v.device, dtype=torch.float32)
+    gates = (MEMORY_KINDS[kind], ga, gb, a_log, dt_bias, log_decay, skip)
+    if b.Tp:
+        n = b.p_ctx.shape[0]
+        plan = _memory_plan(b, v.device)
+        if plan is None:
+            nat.memory_chunks(q, k, v, *gates, S, b.state[:n], b.cu[:n + 1], b.start[:n], None, out, b.Tp)
+        else:
+            pcu, base, P = plan
+            f32 = dict(dtype=torch.float32, device=v.device)
+            loc = torch.empty(P, H, dk, dv, **f32)
+            dec = torch.empty(P, H, **f32)
+            dkp = (dk + 15) // 16 * 16
+            trans = torch.empty(P, H, dkp, dkp, **f32) if kind == "delta" else None
+            init = torch.empty(P, H, dk, dv, **f32)
+            nat.memory_chunk_local(q, k, v, *gates, pcu, loc, dec, trans)
+            nat.memory_combine(S, b.state[:n], b.start[:n], base, loc, dec, trans, init)
+            nat.memory_chunks(q, k, v, *gates, S, None, pcu, None, init, out, b.Tp)
+    if T > b.Tp:
+        n0 = b.cu.shape[0] - 1 - (T - b.Tp)
+        nat.memory_decode(q, k, v, *gates, S, b.state[n0:], b.start[n0:], out, b.Tp)
+    return out
+
+
+def gate_groupnorm(o, z, w, groups: int, eps: float, out_dtype):
+    """``y = o silu(z)`` (o fp32 ``[T, C]``, z ``[T, C]``), then an RMS norm of y in ``groups`` equal consecutive parts, each
+    over its own root mean square, the whole times ``w [C]``: the gate comes before the norm."""
+    if use_native(o):
+        return native_hybrid().gate_groupnorm(o, z, w, groups, eps, out_dtype == torch.bfloat16)
+    return ref.gate_groupnorm(o, z, w, groups, eps, out_dtype)
+
+
+def norm_add_f32_(x, y1, s1: float, y2, s2: float, w, mult: float, eps: float, one_plus: bool, out_dtype):
+    """The end of a sublayer whose only norm is on its result: ``y = s1 y1 (+ s2 y2)``, ``x += mult y / rms(y) (w + one_plus)``
+    in place on the fp32 stream, and the next sublayer's input, x itself, in ``out_dtype``.  ``y [T, W]`` in the activation
+    dtype (row-strided views allowed)."""
+    if use_native(x):
+        return native_hybrid().norm_add_f32_(x, y1, s1, y2, s2, w, mult, eps, one_plus, out_dtype == torch.bfloat16)
+    return ref.norm_add_f32_(x, y1, s1, y2, s2, w, mult, eps, one_plus, out_dtype)
+
+
+def embed_f32(ids, table):
+    """The embedding rows as the fp32 residual stream and in the table's dtype: (x, h)."""
+    if use_native(table):
+        return native_hybrid().embed_f32(ids, table)
+    return ref.embed_f32(ids, table)

@@ -233,7 +233,8 @@ def headnorm_gate(o, w, g, eps, out_dtype, silu=False):
     y = of * torch.rsqrt(of.pow(2).mean(-1, keepdim=True) + eps)
     gf = g.float()
     gate = gf * torch.sigmoid(gf) if silu else torch.sigmoid(gf)
-    return (y.reshape(T, H * dv) * w.float() * gate).to(out_dtype)
+    y = y.reshape(T, H * dv)
+    return ((y if w is None else y * w.float()) * gate).to(out_dtype)
 
 
 def group_topk_router(logits, top, groups, keep):
@@ -296,10 +297,11 @@ def gla_scan(q, k, v, z, z_bias, tau, qscale, S, state_slots, cu, start):
     return out
 
 
-def qk_fullnorm_prep(z, H, G, dk, dv, q_norm, k_norm, eps, pos, temp_coef, temp_every, cache, slots):
+def qk_fullnorm_prep(z, H, G, dk, dv, q_norm, k_norm, eps, pos, temp_coef, temp_every, cache, slots, freq=None, rot_dims=0,
+                     interleaved=False, amp=1.0):
     """z [T, >= H*dk + G*dk + G*dv] = [q | k | v | ...]: RMS norm of all of q and of all of k (weights [H*dk],
-    [G*dk]); q times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1); k and v go to the token's cache row
-    [G, dv + dk] = [v | k]; returns q [T, H, dk]."""
+    [G*dk]); q times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1); rotary of q and k on the first ``rot_dims``
+    entries of every head; k and v go to the token's cache row [G, dv + dk] = [v | k]; returns q [T, H, dk]."""
     T = z.shape[0]
     zf = z.float()
     unit = lambda x: x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
@@ -308,6 +310,9 @@ def qk_fullnorm_prep(z, H, G, dk, dv, q_norm, k_norm, eps, pos, temp_coef, temp_
     v = zf[:, (H + G) * dk:(H + G) * dk + G * dv].view(T, G, dv)
     if temp_coef != 0.0:
         q = q * (1.0 + temp_coef * torch.log(torch.floor((pos.float() + 1.0) / float(temp_every)) + 1.0))[:, None]
+    if rot_dims:
+        q = _rotate(q.view(T, H, dk), pos, freq, rot_dims, interleaved, amp)
+        k = _rotate(k.view(T, G, dk), pos, freq, rot_dims, interleaved, amp)
     row = torch.cat([v, k.view(T, G, dk)], -1).reshape(T, G * (dv + dk)).to(cache.dtype)
     ok = slots >= 0
     cache.view(-1, cache.shape[-1])[slots[ok]] = row[ok]
@@ -468,3 +473,82 @@ def diff_attention(q, cache, bt, cu, ctx, heads, groups, dk, dv, window, scale, 
         o[a:b] = m[0] - lam.float().reshape(()) * m[1]
     o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * post
     out.copy_(o.reshape(n_rows, heads * dv).to(out.dtype))
+
+
+def conv_silu_unit(u, w, bias, state, cu, start, sslot, nq, nk, dk, qscale, eps):
+    """silu(causal convolution + bias) of the packed rows u [T, C]; the first ``nq`` and the next ``nk`` groups of ``dk``
+    channels become unit vectors (q ones times ``qscale``), fp32 [T, nq + nk, dk]; the other channels keep u's dtype."""
+    T = u.shape[0]
+    y = causal_conv(u.float(), w, state, None, cu, start, sslot, False)
+    if bias is not None:
+        y = y + bias.float()
+    y = (y * torch.sigmoid(y)).to(u.dtype)
+    n = (nq + nk) * dk
+    if n == 0:
+        return None, y
+    qk = y[:, :n].float().view(T, nq + nk, dk)
+    qk = qk / torch.sqrt(qk.pow(2).sum(-1, keepdim=True) + eps)
+    qk[:, :nq] *= qscale
+    return qk, y[:, n:]
+
+
+def rotary_f32(z, nq, nk, dk, pos, freq, rot_dims, interleaved, amp, kscale):
+    x = _rotate(z[:, :(nq + nk) * dk].float().reshape(z.shape[0], nq + nk, dk), pos, freq, rot_dims, interleaved, amp)
+    return torch.cat([x[:, :nq], x[:, nq:] * kscale], 1)
+
+
+def memory_gates(kind, T, H, ga, gb, a_log, dt_bias, log_decay):
+    """(log decay, write strength) fp32 [T, H] of :func:`memory_scan`."""
+    if kind == "fixed":
+        return log_decay.float()[None, :].expand(T, H), torch.ones(T, H)
+    dt = torch.nn.functional.softplus(ga.float() + dt_bias.float(), threshold=1e30)
+    la = -torch.exp(a_log.float()) * dt
+    return la, (dt if kind == "ssm" else torch.sigmoid(gb.float()))
+
+
+def memory_scan(q, k, v, kind, ga, gb, a_log, dt_bias, log_decay, skip, S, state_slots, cu, start):
+    """Token by token: S <- g S; u = beta (v - S^T k) (kind "delta") or beta v; S <- S + k u^T; o = S^T q (+ skip v).  The
+    state pool S [slots, H, dk, dv] (fp32) is read at ``state_slots[seq]`` (zeros when the sequence starts at position
+    0) and written back after the sequence's last token of this step."""
+    T, H, dv = v.shape
+    rep = H // q.shape[1]
+    q, k, v = q.float().repeat_interleave(rep, 1), k.float().repeat_interleave(rep, 1), v.float()
+    la, beta = memory_gates(kind, T, H, ga, gb, a_log, dt_bias, log_decay)
+    g = torch.exp(la)
+    out = torch.zeros(T, H, dv)
+    cu_l = [int(x) for x in cu]
+    for s in range(len(cu_l) - 1):
+        if cu_l[s] == cu_l[s + 1]:
+            continue
+        slot = int(state_slots[s])
+        St = torch.zeros_like(S[slot]) if int(start[s]) == 0 else S[slot].clone()
+        for t in range(cu_l[s], cu_l[s + 1]):
+            St = g[t][:, None, None] * St
+            u = v[t]
+            if kind == "delta":
+                u = u - torch.einsum("hkv,hk->hv", St, k[t])
+            u = beta[t][:, None] * u
+            St = St + k[t][:, :, None] * u[:, None, :]
+            out[t] = torch.einsum("hkv,hk->hv", St, q[t])
+        S[slot] = St
+    return out if skip is None else out + skip.float()[None, :, None] * v
+
+
+def gate_groupnorm(o, z, w, groups, eps, out_dtype):
+    zf = z.float()
+    y = o.float() * zf * torch.sigmoid(zf)
+    p = y.view(y.shape[0], groups, -1)
+    return ((p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)).reshape(y.shape) * w.float()).to(out_dtype)
+
+
+def norm_add_f32_(x, y1, s1, y2, s2, w, mult, eps, one_plus, out_dtype):
+    y = y1.float() * s1
+    if y2 is not None:
+        y = y + y2.float() * s2
+    x += mult * (y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps) * (w.float() + (1.0 if one_plus else 0.0)))
+    return x.to(out_dtype) if out_dtype != torch.float32 else x.clone()
+
+
+def embed_f32(ids, table):
+    h = table[ids]
+    return h.float().clone(), h
