@@ -77,13 +77,19 @@ def parse():
                     help="instead of the training benchmark: serving prefill / decode throughput of Pamazen "
                          "configurations beside Malinex at equal size (comma-separated sizes of "
                          "llmctl.benchmarks.hybrid.PAMAZEN_SIZES, or 'all'); one JSON line per size")
+    ap.add_argument("--dumazen-compare", default=None, metavar="SIZES",
+                    help="instead of the training benchmark: serving prefill / decode throughput of Dumazen "
+                         "configurations beside Malinex at equal size (comma-separated sizes of "
+                         "llmctl.benchmarks.hybrid.DUMAZEN_SIZES, or 'all'); one JSON line per size")
     return ap.parse_args()
 
 
 def hybrid_compare(args) -> None:
     from llmctl.benchmarks import hybrid
 
-    if args.dapipel_compare:
+    if args.dumazen_compare:
+        table, which, family = hybrid.DUMAZEN_SIZES, args.dumazen_compare, "dumazen"
+    elif args.dapipel_compare:
         table, which, family = hybrid.DAPIPEL_SIZES, args.dapipel_compare, "dapipel"
     elif args.pamazen_compare:
         table, which, family = hybrid.PAMAZEN_SIZES, args.pamazen_compare, "pamazen"
@@ -100,7 +106,7 @@ def hybrid_compare(args) -> None:
 
 def main():
     args = parse()
-    if args.hybrid_compare or args.dumalix_compare or args.malinex_compare or args.pamazen_compare or args.dapipel_compare:
+    if args.hybrid_compare or args.dumalix_compare or args.malinex_compare or args.pamazen_compare or args.dapipel_compare or args.dumazen_compare:
         return hybrid_compare(args)
     import torch
     import torch.distributed as dist

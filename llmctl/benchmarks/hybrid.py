@@ -8,7 +8,9 @@ closest existing model: grouped-query attention over paged rows beside a decayed
 softmax-routed experts with a shared one, an fp32 residual stream) at equal width, depth, heads, kv heads, experts
 and expert size, and of a Dapipel configuration beside Malinex (the closest existing model: a recurrence over state
 slots in two layers of three, grouped-query attention over paged rows in the third, learned positions) at equal width,
-depth, heads, kv heads and feed-forward.
+depth, heads, kv heads and feed-forward, and of a Dumazen configuration beside Malinex (the closest existing model: matrix
+memories in state slots in two layers of three, grouped-query attention over paged rows in the third) at equal width, depth,
+heads, kv heads, memory sizes and dense feed-forward.
 
 Both run through the same engine calls: one prompt portion per sequence (``InferenceEngine.prefill``)
 and then one-token decode steps of the whole batch (``InferenceEngine.decode``); random weights,
@@ -73,6 +75,27 @@ DAPIPEL_SIZES = {
     "medium-dense": dict(width=2048, layers=6, heads=16, kv_heads=4, head_dim=128, experts=0, top=0, ff=4096, window=1024, prompt=2048, batch=16),
     "large-dense": dict(width=4096, layers=6, heads=32, kv_heads=8, head_dim=128, experts=0, top=0, ff=8192, window=1024, prompt=4096, batch=16),
 }
+
+
+# Dumazen: width, layers (every third is the pair of windowed attention and gated delta rule, the others Mamba-2 and retention by
+# turns), heads of ``head_dim`` (memories: keys of half that), kv heads, ungated feed-forward, window, prompt, decode batch
+DUMAZEN_SIZES = {
+    "tiny": dict(width=128, layers=3, heads=4, kv_heads=2, head_dim=32, ff=256, window=32, prompt=160, batch=2),
+    "small": dict(width=1024, layers=6, heads=8, kv_heads=2, head_dim=128, ff=4096, window=1024, prompt=2048, batch=16),
+    "medium": dict(width=2048, layers=6, heads=16, kv_heads=4, head_dim=128, ff=8192, window=1024, prompt=2048, batch=16),
+    "large": dict(width=4096, layers=6, heads=32, kv_heads=8, head_dim=128, ff=16384, window=1024, prompt=4096, batch=16),
+}
+
+
+def _configs_dumazen(s: Dict):
+    from llmctl.models.dumazen import dumazen_template
+    from llmctl.models.malinex import malinex_template
+
+    kw = dict(width=s["width"], layers=s["layers"], heads=s["heads"], kv_heads=s["kv_heads"], vocab=32000, every=3, ff=s["ff"],
+              head_dim=s["head_dim"])
+    du = dumazen_template(window=s["window"], **kw)
+    du.max_position_embeddings = s["prompt"] + 256
+    return du, malinex_template(experts=0, max_positions=s["prompt"] + 256, **kw)
 
 
 def _configs_dapipel(s: Dict):
@@ -202,7 +225,12 @@ def _measure(eng, prompt: int, batch: int, steps: int, warmup: int) -> Dict[str,
 def run(sizes: List[str], device: str = "auto", steps: int = 5, warmup: int = 2, family: str = "lenitar") -> List[Dict]:
     out = []
     for name in sizes:
-        if family == "dapipel":
+        if family == "dumazen":
+            s = DUMAZEN_SIZES[name]
+            hy, tr = _configs_dumazen(s)
+            row = {"size": name, **s}
+            pair = (("dumazen", hy), ("malinex", tr))
+        elif family == "dapipel":
             s = DAPIPEL_SIZES[name]
             hy, tr = _configs_dapipel(s)
             row = {"size": name, **s}

@@ -272,7 +272,7 @@ def dumazen_template(width: int = 256, layers: int = 4, heads: int = 4, kv_heads
     d = head_dim or width // heads
     dk = max(d // 2 // 2 * 2, 2)
     par = {"left": {"heads": heads, "kv_heads": kv_heads, "dim": d, "vdim": d, "scale": d ** -0.5, "mask": {"size": window},
-                    "rot": {"base": 500000.0, "dims": d // 2 * 2, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+                    "rot": {"base": 100000.0, "dims": d // 2 * 2, "scaling": {"factor": 4.0, "low": 1.0, "high": 4.0, "original": 8192}}},
            "right": {"heads": heads, "kv_heads": heads, "dim": dk, "vdim": d, "conv": taps}, "left_scale": 0.5, "right_scale": 0.5}
     ssm = {"heads": heads, "vdim": d, "state": dk, "groups": 1, "conv": taps, "norm_groups": 1}
     ret = {"heads": heads, "dim": dk, "vdim": d, "rot": {"base": 10000.0, "dims": dk},

@@ -43,11 +43,10 @@ def conv(u, w, bias=None):
     """sum_j w[:, j] u_(t - taps + 1 + j) (+ bias) per channel, zeros before the first row."""
     T, taps = u.shape[0], w.shape[1]
     out = torch.zeros_like(u)
-    for t in range(T):
-        for j in range(taps):
-            s = t - taps + 1 + j
-            if s >= 0:
-                out[t] = out[t] + w[:, j] * u[s]
+    for j in range(taps):
+        back = taps - 1 - j
+        for t in range(back, T):
+            out[t] += w[:, j] * u[t - back]
     return out if bias is None else out + bias
 
 
@@ -74,12 +73,12 @@ def frequencies(rot):
 def rotate(x, rot):
     """x [T, n]: entry i of the first ``dims`` is turned with entry i + dims/2 by position * f_i."""
     half = int(rot["dims"]) // 2
+    t = torch.arange(x.shape[0], dtype=F64)
     y = x.clone()
-    for t in range(x.shape[0]):
-        for i, f in enumerate(frequencies(rot)):
-            c, s = math.cos(t * f), math.sin(t * f)
-            u, v = x[t, i], x[t, i + half]
-            y[t, i], y[t, i + half] = u * c - v * s, v * c + u * s
+    for i, f in enumerate(frequencies(rot)):
+        c, s = torch.cos(t * f), torch.sin(t * f)
+        u, v = x[:, i], x[:, i + half]
+        y[:, i], y[:, i + half] = u * c - v * s, v * c + u * s
     return y
 
 
@@ -112,9 +111,28 @@ def unit(x):
     return x / torch.sqrt((x * x).sum(-1, keepdim=True) + 1e-6)
 
 
+def delta_memory(q, k, v, decay, beta, S):
+    """One head over T tokens from memory S [dim, vdim]: (outputs [T, vdim], the memory after the last token)."""
+    rows = []
+    for t in range(v.shape[0]):
+        S = decay[t] * S
+        u = beta[t] * (v[t] - S.T @ k[t])
+        S = S + torch.outer(k[t], u)
+        rows.append(S.T @ q[t])
+    return torch.stack(rows), S
+
+
+def decayed_memory(q, k, v, decay, write, S):
+    """The same without the subtraction: every token adds ``write`` times k v^T."""
+    rows = []
+    for t in range(v.shape[0]):
+        S = decay[t] * S + write[t] * torch.outer(k[t], v[t])
+        rows.append(S.T @ q[t])
+    return torch.stack(rows), S
+
+
 def delta_rule(h, W, p, m, eps):
     """The gated delta rule: decay the memory, write the part of v that it does not give for k, read with q."""
-    T = h.shape[0]
     H, G, d, dv = int(m["heads"]), int(m.get("kv_heads", m["heads"])), int(m["dim"]), int(m["vdim"])
     q, k, v = (silu(conv(h @ W[p + n].T, W[p + n + ".conv"])) for n in ("q", "k", "v"))
     beta = sigmoid(h @ W[p + "b"].T)
@@ -123,13 +141,8 @@ def delta_rule(h, W, p, m, eps):
     for n in range(H):
         g = n // (H // G)
         qn, kn = unit(q[:, g * d:(g + 1) * d]) * d ** -0.5, unit(k[:, g * d:(g + 1) * d])
-        S, rows = torch.zeros(d, dv, dtype=F64), []
-        for t in range(T):
-            S = decay[t, n] * S
-            u = beta[t, n] * (v[t, n * dv:(n + 1) * dv] - S.T @ kn[t])
-            S = S + torch.outer(kn[t], u)
-            rows.append(S.T @ qn[t])
-        heads.append(rms(torch.stack(rows), eps) * W[p + "norm"])
+        o, _ = delta_memory(qn, kn, v[:, n * dv:(n + 1) * dv], decay[:, n], beta[:, n], torch.zeros(d, dv, dtype=F64))
+        heads.append(rms(o, eps) * W[p + "norm"])
     return (torch.cat(heads, -1) * silu(h @ W[p + "g"].T)) @ W[p + "o"].T
 
 
@@ -139,7 +152,6 @@ def parallel(h, W, p, m, eps):
 
 
 def mamba2(h, W, p, m, eps):
-    T = h.shape[0]
     H, dv, N, G = int(m["heads"]), int(m["vdim"]), int(m["state"]), int(m["groups"])
     inner = H * dv
     z, xbc, dt = torch.split(h @ W[p + "in"].T, [inner, inner + 2 * G * N, H], -1)
@@ -149,12 +161,10 @@ def mamba2(h, W, p, m, eps):
     heads = []
     for n in range(H):
         g = n // (H // G)
-        S, rows = torch.zeros(N, dv, dtype=F64), []
-        for t in range(T):
-            xt = x[t, n * dv:(n + 1) * dv]
-            S = torch.exp(-torch.exp(W[p + "A_log"][n]) * dt[t, n]) * S + dt[t, n] * torch.outer(B[t, g * N:(g + 1) * N], xt)
-            rows.append(S.T @ C[t, g * N:(g + 1) * N] + W[p + "D"][n] * xt)
-        heads.append(torch.stack(rows))
+        xn, cols = x[:, n * dv:(n + 1) * dv], slice(g * N, (g + 1) * N)
+        decay = torch.exp(-torch.exp(W[p + "A_log"][n]) * dt[:, n])
+        o, _ = decayed_memory(C[:, cols], B[:, cols], xn, decay, dt[:, n], torch.zeros(N, dv, dtype=F64))
+        heads.append(o + W[p + "D"][n] * xn)
     y = torch.cat(heads, -1) * silu(z)
     part = inner // int(m["norm_groups"])
     y = torch.cat([rms(y[:, i:i + part], eps) for i in range(0, inner, part)], -1) * W[p + "norm"]
@@ -168,11 +178,9 @@ def retention(h, W, p, m, eps):
     heads = []
     for n in range(H):
         qn, kn = rotate(q[:, n * d:(n + 1) * d], m["rot"]), rotate(k[:, n * d:(n + 1) * d], m["rot"]) * d ** -0.5
-        S, rows = torch.zeros(d, dv, dtype=F64), []
-        for t in range(T):
-            S = float(m["decay"][n]) * S + torch.outer(kn[t], v[t, n * dv:(n + 1) * dv])
-            rows.append(S.T @ qn[t])
-        heads.append(rms(torch.stack(rows), eps))
+        one = torch.ones(T, dtype=F64)
+        o, _ = decayed_memory(qn, kn, v[:, n * dv:(n + 1) * dv], float(m["decay"][n]) * one, one, torch.zeros(d, dv, dtype=F64))
+        heads.append(rms(o, eps))
     return (torch.cat(heads, -1) * silu(h @ W[p + "g"].T)) @ W[p + "o"].T
 
 
