@@ -790,9 +790,9 @@ class GatedDeltaRule(nn.Module):
             z = F.linear(h, self.w_in)
         c, g0 = self.conv.channels, self.conv.channels + H * dv
         qk, v = hops.conv_silu_unit(z[:, :c], self.conv.tap_major(), None, carried, b, G, G, self.dk, self.dk ** -0.5, self.key_eps)
-        o = hops.memory_scan(qk[:, :G], qk[:, G:], v.unflatten(1, (H, dv)), "delta", S, b, ga=z[:, g0:g0 + H],
-                             gb=z[:, g0 + H:g0 + 2 * H], a_log=self.a_log, dt_bias=self.dt_bias)
-        return F.linear(hops.headnorm_gate(o, self._norm_rows(), z[:, c:g0], self.eps, h.dtype, silu=True), self.w_o)
+        y = hops.memory_scan(qk[:, :G], qk[:, G:], v.view(-1, H, dv), "delta", S, b, ga=z[:, g0:g0 + H], gb=z[:, g0 + H:g0 + 2 * H],
+                             a_log=self.a_log, dt_bias=self.dt_bias, norm=(self._norm_rows(), z[:, c:g0], self.eps))
+        return F.linear(y, self.w_o)
 
 
 class Mamba2(nn.Module):
@@ -881,8 +881,9 @@ class Retention(nn.Module):
         z = F.linear(h, self.w_in)
         qk = hops.rotary_f32(z, H, H, dk, b.pos, self.inv_freq, self.rot_dims, self.interleaved, self.rot_amp, dk ** -0.5)
         v0, g0 = 2 * H * dk, 2 * H * dk + H * dv
-        o = hops.memory_scan(qk[:, :H], qk[:, H:], z[:, v0:g0].unflatten(1, (H, dv)), "fixed", S, b, log_decay=self.log_decay)
-        return F.linear(hops.headnorm_gate(o, None, z[:, g0:g0 + H * dv], self.eps, h.dtype, silu=True), self.w_o)
+        y = hops.memory_scan(qk[:, :H], qk[:, H:], z[:, v0:g0].unflatten(1, (H, dv)), "fixed", S, b, log_decay=self.log_decay,
+                             norm=(None, z[:, g0:g0 + H * dv], self.eps))
+        return F.linear(y, self.w_o)
 
 
 class ParallelMixers(nn.Module):

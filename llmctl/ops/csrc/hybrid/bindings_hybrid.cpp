@@ -95,10 +95,10 @@ std::tuple<at::Tensor, at::Tensor> conv_silu_unit(const at::Tensor& u, const at:
 using OptT = c10::optional<at::Tensor>;
 void memory_decode(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, int64_t kind, const OptT& ga, const OptT& gb, const OptT& a_log,
                    const OptT& dt_bias, const OptT& log_decay, const OptT& skip, at::Tensor S, const at::Tensor& slots, const at::Tensor& start,
-                   at::Tensor out, int64_t row0);
+                   at::Tensor out, const OptT& hn_w, const OptT& hn_g, double hn_eps, int64_t row0);
 void memory_chunks(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, int64_t kind, const OptT& ga, const OptT& gb, const OptT& a_log,
                    const OptT& dt_bias, const OptT& log_decay, const OptT& skip, at::Tensor S, const OptT& slots, const at::Tensor& cu,
-                   const OptT& start, const OptT& init, at::Tensor out, int64_t rows);
+                   const OptT& start, const OptT& init, at::Tensor out, const OptT& hn_w, const OptT& hn_g, double hn_eps, int64_t rows);
 void memory_chunk_local(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, int64_t kind, const OptT& ga, const OptT& gb, const OptT& a_log,
                         const OptT& dt_bias, const OptT& log_decay, const OptT& skip, const at::Tensor& cu, at::Tensor loc, at::Tensor dec,
                         const OptT& trans);
@@ -153,8 +153,8 @@ TORCH_LIBRARY(llmctl_hybrid, m) {
   m.def("kv_rows_write(Tensor k, Tensor v, Tensor(a!) cache, Tensor slots, int groups) -> ()");
   m.def("diff_attn(Tensor q, Tensor cache, Tensor bt, Tensor? cu, Tensor ctx, int heads, int groups, int dk, int dv, int window, float scale, Tensor lam, float post, float eps, int max_q, int max_ctx, bool mfma, Tensor(a!) out) -> ()");
   m.def("conv_silu_unit(Tensor u, Tensor w, Tensor? bias, Tensor(a!) state, Tensor seq_of, Tensor cu, Tensor start, Tensor sslot, int nq, int nk, int dk, float qscale, float eps, int max_len=0) -> (Tensor, Tensor)");
-  m.def("memory_decode(Tensor q, Tensor k, Tensor v, int kind, Tensor? ga, Tensor? gb, Tensor? a_log, Tensor? dt_bias, Tensor? log_decay, Tensor? skip, Tensor(a!) S, Tensor slots, Tensor start, Tensor(b!) out, int row0) -> ()");
-  m.def("memory_chunks(Tensor q, Tensor k, Tensor v, int kind, Tensor? ga, Tensor? gb, Tensor? a_log, Tensor? dt_bias, Tensor? log_decay, Tensor? skip, Tensor(a!) S, Tensor? slots, Tensor cu, Tensor? start, Tensor? init, Tensor(b!) out, int rows) -> ()");
+  m.def("memory_decode(Tensor q, Tensor k, Tensor v, int kind, Tensor? ga, Tensor? gb, Tensor? a_log, Tensor? dt_bias, Tensor? log_decay, Tensor? skip, Tensor(a!) S, Tensor slots, Tensor start, Tensor(b!) out, Tensor? hn_w, Tensor? hn_g, float hn_eps, int row0) -> ()");
+  m.def("memory_chunks(Tensor q, Tensor k, Tensor v, int kind, Tensor? ga, Tensor? gb, Tensor? a_log, Tensor? dt_bias, Tensor? log_decay, Tensor? skip, Tensor(a!) S, Tensor? slots, Tensor cu, Tensor? start, Tensor? init, Tensor(b!) out, Tensor? hn_w, Tensor? hn_g, float hn_eps, int rows) -> ()");
   m.def("memory_chunk_local(Tensor q, Tensor k, Tensor v, int kind, Tensor? ga, Tensor? gb, Tensor? a_log, Tensor? dt_bias, Tensor? log_decay, Tensor? skip, Tensor cu, Tensor(a!) loc, Tensor(b!) dec, Tensor(c!)? trans) -> ()");
   m.def("memory_combine(Tensor(a!) S, Tensor slots, Tensor start, Tensor base, Tensor loc, Tensor dec, Tensor? trans, Tensor(b!) init) -> ()");
   m.def("embed_f32(Tensor ids, Tensor table) -> (Tensor, Tensor)");

@@ -202,6 +202,9 @@ struct ConvUnitArgs {
   float qscale, eps;
 };
 
+constexpr int CONV_WALK = 8;  // tokens per walk at most (CONV_SHORT fits)
+static_assert(CONV_SHORT <= CONV_WALK, "short portions are one walk");
+
 // A unit is a group of dk channels, or a span of lg * VEC * NI of the other channels.  TAPS == 0: any number of taps.
 template <typename T, int VEC, int NI, int TAPS>
 __global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
@@ -269,11 +272,21 @@ __global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
     }
   }
   float hist[NH][NI][VEC];  // hist[k]: the input k + 1 positions before the current token
+  float in[CONV_WALK][NI][VEC];  // the walk's inputs, requested at once
+#pragma unroll
+  for (int j = 0; j < CONV_WALK; ++j)
+    if (t_lo + j < t_hi) {
+#pragma unroll
+      for (int i = 0; i < NI; ++i) load_row(u + (int64_t)(t_lo + j) * a.u_st + ch[i], in[j][i]);
+    }
   int s = a.whole ? (int)blockIdx.x : a.seq_of[t_lo];
   int s0 = a.cu[s], s1 = a.cu[s + 1], p0 = a.start[s];
   float* st = a.state + (int64_t)a.sslot[s] * (taps - 1) * a.C;
-  for (int t = t_lo; t < t_hi; ++t) {
-    bool reload = t == t_lo;
+#pragma unroll
+  for (int jt = 0; jt < CONV_WALK; ++jt) {
+    const int t = t_lo + jt;
+    if (t >= t_hi) break;
+    bool reload = jt == 0;
     if (t >= s1) {
       s = a.seq_of[t];
       s0 = a.cu[s], s1 = a.cu[s + 1], p0 = a.start[s];
@@ -291,8 +304,7 @@ __global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
     float x[NI][VEC], ss = 0.f;
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      float cur[VEC];
-      load_row(u + (int64_t)t * a.u_st + ch[i], cur);
+      const float(&cur)[VEC] = in[jt][i];
       if constexpr (TAPS > 0) {
 #pragma unroll
         for (int c = 0; c < VEC; ++c) {
@@ -323,7 +335,7 @@ __global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
       }
 #pragma unroll
       for (int c = 0; c < VEC; ++c) {
-        x[i][c] = x[i][c] / (1.0f + expf(-x[i][c]));
+        x[i][c] *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x[i][c]));  // silu
         if (ok[i]) ss += x[i][c] * x[i][c];
       }
     }
@@ -412,8 +424,8 @@ std::tuple<at::Tensor, at::Tensor> conv_silu_unit(const at::Tensor& u, const at:
   const int NIv = ni > 1 ? 4 : 1;
   const int64_t span = (int64_t)lg * vec * NIv, units = ng + (C - ng * dk + span - 1) / span;
   const int64_t by = (units * lg + 255) / 256;
-  a.tok = 1;  // tokens per walk: as many as leave the chip a few thousand workgroups
-  while (a.tok < 16 && T * by / (2 * a.tok) >= 2048) a.tok *= 2;
+  a.tok = 1;  // tokens per walk: as many as leave the chip a thousand workgroups
+  while (a.tok < CONV_WALK && T * by / (2 * a.tok) >= 1024) a.tok *= 2;
   HYB_CHECK(by <= 65535, "too many channels for one launch");
   const dim3 grid((unsigned)(a.whole ? ns : (T + a.tok - 1) / a.tok), (unsigned)by);
   dispatch_act(u, [&](auto* tag) {

@@ -10,6 +10,7 @@
 //                        u solve (I + A) U = beta (V - e^L K S_0) with A_ts = beta_t e^(L_t - L_s) (k_t . k_s), s < t, block by
 //                        block (16 x 16 diagonal blocks are inverted by substitution).  Called on whole portions it also
 //                        writes the new memory, e^(L_n) S_0 + sum_t e^(L_n - L_t) k_t u_t^T.
+//                        Both of these can end in the mixer's head norm: o over its root mean square, a weight, a silu gate.
 //   memory_chunk_local   every chunk from a zero memory: its own contribution, its total decay and, for the delta kind, the
 //                        matrix that carries a memory over the chunk (the same solve on the columns of K)
 //   memory_combine       the memory at every chunk's first token in order, and the sequence's new carried memory
@@ -51,32 +52,42 @@ struct MemArgs {
   float* dec;         // [chunks, H]
   float* trans;       // [chunks, H, dkp, dkp]
   float* out;         // [T, H, dv]
+  // fused head norm (y given, out not): y = o / rms(o over dv) * hn_w (if given) * hn_g sigmoid(hn_g), [T, H * dv] in v's dtype
+  void* y;
+  const float* hn_w;  // nullptr or [H * dv]
+  const void* hn_g;   // [T, H * dv] in v's dtype
+  int64_t hn_st;
+  float hn_eps;
   int kind, H, rep, dk, dv, vec, row0;
 };
 
-template <typename TV>
-__device__ __forceinline__ void gates(const MemArgs& a, int h, int64_t t, float& la, float& beta) {
+// z sigmoid(z); the hardware's exponential and reciprocal are good to an ulp
+__device__ __forceinline__ float silu(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)); }
+
+// (log g, beta) of head h from the raw gate columns
+__device__ __forceinline__ void gate_values(const MemArgs& a, int h, float ga, float gb, float& la, float& beta) {
   if (a.kind == KIND_FIXED) {
     la = a.log_decay[h];
     beta = 1.0f;
     return;
   }
-  const float x = ldf(reinterpret_cast<const TV*>(a.ga) + t * a.ga_st + h) + a.dt_bias[h];
+  const float x = ga + a.dt_bias[h];
   const float dt = fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
   la = -expf(a.a_log[h]) * dt;
-  beta = a.kind == KIND_SSM ? dt : 1.0f / (1.0f + expf(-ldf(reinterpret_cast<const TV*>(a.gb) + t * a.gb_st + h)));
+  beta = a.kind == KIND_SSM ? dt : 1.0f / (1.0f + expf(-gb));
 }
 
 // ------------------------------------------------------------------------------------------ decode
-// 16 thread groups share the dk rows of S; a thread owns VEC neighbouring value columns of its rows.
-template <typename TQ, typename TV, int VEC, int NR>
-__global__ __launch_bounds__(256) void memory_decode_kernel(MemArgs a) {
-  __shared__ float red[4][16][2 * VEC + 1];
+// 16 thread groups share the dk rows of S; a thread owns VEC neighbouring value columns of its rows, CL threads a row.
+template <typename TQ, typename TV, int VEC, int NR, int CL>
+__global__ __launch_bounds__(16 * CL) void memory_decode_kernel(MemArgs a) {
+  constexpr int NWV = 16 * CL / 64, NS = 2 * VEC + 1;
+  __shared__ float red[NWV][CL][NS];
   const int n = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
-  const int wave = tid >> 6, cl = tid & 15, rg = tid >> 4;
+  const int wave = tid >> 6, cl = tid % CL, rg = tid / CL;
   const int64_t t = a.row0 + n;
   const int dk = a.dk, dv = a.dv;
-  const int col = blockIdx.z * 16 * VEC + cl * VEC;
+  const int col = blockIdx.z * CL * VEC + cl * VEC;
   const bool cok = col < dv;  // VEC divides dv
   const int colc = cok ? col : 0;
   const TQ* qp = reinterpret_cast<const TQ*>(a.q) + t * a.q_st + (h / a.rep) * a.q_sh;
@@ -84,7 +95,7 @@ __global__ __launch_bounds__(256) void memory_decode_kernel(MemArgs a) {
   const TV* vp = reinterpret_cast<const TV*>(a.v) + t * a.v_st + h * a.v_sh + colc;
   float* Sb = a.S + ((int64_t)a.slots[n] * a.H + h) * dk * dv + colc;
   const bool fresh = a.start[n] == 0;
-  float S[NR][VEC], kr[NR], qr[NR], v[VEC];
+  float S[NR][VEC], kr[NR], qr[NR], v[VEC], gt[VEC];
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
     const int d = rg + 16 * i;
@@ -99,13 +110,17 @@ __global__ __launch_bounds__(256) void memory_decode_kernel(MemArgs a) {
     qr[i] = ok ? ldf(qp + d) : 0.f;
   }
 #pragma unroll
-  for (int c = 0; c < VEC; ++c) v[c] = ldf(vp + c);
+  for (int c = 0; c < VEC; ++c) {
+    v[c] = ldf(vp + c);
+    gt[c] = a.y != nullptr ? ldf(reinterpret_cast<const TV*>(a.hn_g) + t * a.hn_st + h * dv + colc + c) : 0.f;
+  }
   float la, beta;
-  gates<TV>(a, h, t, la, beta);
+  gate_values(a, h, a.kind != KIND_FIXED ? ldf(reinterpret_cast<const TV*>(a.ga) + t * a.ga_st + h) : 0.f,
+              a.kind == KIND_DELTA ? ldf(reinterpret_cast<const TV*>(a.gb) + t * a.gb_st + h) : 0.f, la, beta);
   const float g = expf(la);
-  float sum[2 * VEC + 1];
+  float sum[NS];
 #pragma unroll
-  for (int c = 0; c < 2 * VEC + 1; ++c) sum[c] = 0.f;
+  for (int c = 0; c < NS; ++c) sum[c] = 0.f;
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
 #pragma unroll
@@ -116,36 +131,53 @@ __global__ __launch_bounds__(256) void memory_decode_kernel(MemArgs a) {
     sum[2 * VEC] += kr[i] * qr[i];
   }
 #pragma unroll
-  for (int c = 0; c < 2 * VEC + 1; ++c) {
-    sum[c] += __shfl_xor(sum[c], 16, 64);
-    sum[c] += __shfl_xor(sum[c], 32, 64);
-  }
-  if ((tid & 63) < 16) {
+  for (int c = 0; c < NS; ++c) {
 #pragma unroll
-    for (int c = 0; c < 2 * VEC + 1; ++c) red[wave][cl][c] = sum[c];
+    for (int o = CL; o < 64; o <<= 1) sum[c] += __shfl_xor(sum[c], o, 64);
+  }
+  if ((tid & 63) < CL) {
+#pragma unroll
+    for (int c = 0; c < NS; ++c) red[wave][cl][c] = sum[c];
   }
   __syncthreads();
 #pragma unroll
-  for (int c = 0; c < 2 * VEC + 1; ++c) sum[c] = (red[0][cl][c] + red[1][cl][c]) + (red[2][cl][c] + red[3][cl][c]);
-  if (!cok) return;
+  for (int c = 0; c < NS; ++c) {
+    sum[c] = 0.f;
+#pragma unroll
+    for (int w = 0; w < NWV; ++w) sum[c] += red[w][cl][c];
+  }
   float u[VEC];
 #pragma unroll
   for (int c = 0; c < VEC; ++c) u[c] = beta * (a.kind == KIND_DELTA ? v[c] - g * sum[c] : v[c]);
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
     const int d = rg + 16 * i;
-    if (d < dk) {
+    if (cok && d < dk) {
 #pragma unroll
       for (int c = 0; c < VEC; ++c) S[i][c] = g * S[i][c] + kr[i] * u[c];
       if constexpr (VEC == 4) Vec16<float>::store(Sb + (int64_t)d * dv, S[i]);
       else Sb[(int64_t)d * dv] = S[i][0];
     }
   }
-  if (rg == 0) {
+  if (rg == 0) {  // (CL lanes of the first wave)
     const float sk = a.skip != nullptr ? a.skip[h] : 0.f;
     float o[VEC];
 #pragma unroll
     for (int c = 0; c < VEC; ++c) o[c] = g * sum[VEC + c] + sum[2 * VEC] * u[c] + sk * v[c];
+    if (a.y != nullptr) {  // (one column tile: the lanes hold the whole head)
+      float q = 0.f;
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) q += cok ? o[c] * o[c] : 0.f;
+#pragma unroll
+      for (int x = CL / 2; x > 0; x >>= 1) q += __shfl_xor(q, x, 64);
+      if (!cok) return;
+      const float f = 1.0f / sqrtf(q / (float)dv + a.hn_eps);
+      TV* yp = reinterpret_cast<TV*>(a.y) + (t * a.H + h) * dv + col;
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) stf(yp + c, o[c] * f * (a.hn_w != nullptr ? a.hn_w[h * dv + col + c] : 1.f) * silu(gt[c]));
+      return;
+    }
+    if (!cok) return;
     float* op = a.out + (t * a.H + h) * dv + col;
     if constexpr (VEC == 4) Vec16<float>::store(op, o);
     else op[0] = o[0];
@@ -155,6 +187,15 @@ __global__ __launch_bounds__(256) void memory_decode_kernel(MemArgs a) {
 // ------------------------------------------------------------------------------------------ chunks
 __device__ __forceinline__ f32x4 mfma4(float x, float y, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(x, y, c, 0, 0, 0); }
 __device__ __forceinline__ f32x4 lds4(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+
+// the sum over the 16 lanes of a row, in each of them (rotations inside the row: no LDS)
+__device__ __forceinline__ float sum16(float v) {
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xf, 0xf, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xf, 0xf, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xf, 0xf, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xf, 0xf, true));
+  return v;
+}
 
 // acc += X Y over one 16-wide block: x4 the lane's four A operands, y its four B operands
 __device__ __forceinline__ f32x4 block_product(f32x4 x4, f32x4 y, f32x4 acc) {
@@ -200,13 +241,27 @@ struct ChunkGates {  // LDS arrays of CH floats each
   float* rest;  // e^(L_n - L_t)
 };
 
-// the first wave fills the arrays; tokens past n: no decay, no write
+// The first wave fills the arrays (tokens past n: no decay, no write).  Raw gate values are requested ahead of the rows'
+// staging and used after it.
+struct RawGates {
+  float x, y;
+};
 template <typename TV>
-__device__ __forceinline__ void chunk_gates(const MemArgs& a, const ChunkGates& cg, int h, int t0, int n) {
+__device__ __forceinline__ RawGates load_gates(const MemArgs& a, int h, int t0, int n) {
+  RawGates r = {0.f, 0.f};
+  if ((int)threadIdx.x < n && a.kind != KIND_FIXED) {
+    const int64_t t = t0 + (int)threadIdx.x;
+    r.x = ldf(reinterpret_cast<const TV*>(a.ga) + t * a.ga_st + h);
+    if (a.kind == KIND_DELTA) r.y = ldf(reinterpret_cast<const TV*>(a.gb) + t * a.gb_st + h);
+  }
+  return r;
+}
+
+__device__ __forceinline__ void chunk_gates(const MemArgs& a, const ChunkGates& cg, RawGates raw, int h, int n) {
   if (threadIdx.x < CH) {
     const int t = threadIdx.x;
     float la = 0.f, beta = 0.f;
-    if (t < n) gates<TV>(a, h, t0 + t, la, beta);
+    if (t < n) gate_values(a, h, raw.x, raw.y, la, beta);
     double L = (double)la;
 #pragma unroll
     for (int o = 1; o < CH; o <<= 1) {
@@ -232,7 +287,12 @@ __device__ __forceinline__ void invert_diagonals(const float* A, float* Tb) {
   for (int i = 0; i < 16; ++i) {
     float s = i == j ? 1.f : 0.f;
 #pragma unroll
-    for (int c = 0; c < i; ++c) s -= Ab[i * AS + c] * x[c];
+    for (int c4 = 0; c4 < i; c4 += 4) {
+      const f32x4 a4 = lds4(Ab + i * AS + c4);
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+        if (c4 + c < i) s -= a4[c] * x[c4 + c];
+    }
     x[i] = s;
     Tb[(b * 16 + i) * TBS + j] = s;
   }
@@ -257,11 +317,17 @@ __device__ __forceinline__ void lower_tile(int i, int& ti, int& tj) {  // the te
 }
 
 // one score tile: rows 16 ti .. of X against rows 16 tj .. of Y (both [CH][ks] in LDS)
+template <int NKK>
 __device__ __forceinline__ f32x4 score_tile(const float* X, const float* Y, int ks, int nkk, int ti, int tj, int lane) {
   const float* xr = X + (16 * ti + (lane & 15)) * ks + (lane >> 4) * 4;
   const float* yr = Y + (16 * tj + (lane & 15)) * ks + (lane >> 4) * 4;
   f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-  for (int kk = 0; kk < nkk; ++kk) acc = block_product(lds4(xr + 16 * kk), lds4(yr + 16 * kk), acc);
+  if constexpr (NKK > 0) {
+#pragma unroll
+    for (int kk = 0; kk < NKK; ++kk) acc = block_product(lds4(xr + 16 * kk), lds4(yr + 16 * kk), acc);
+  } else {
+    for (int kk = 0; kk < nkk; ++kk) acc = block_product(lds4(xr + 16 * kk), lds4(yr + 16 * kk), acc);
+  }
   return acc;
 }
 
@@ -282,93 +348,105 @@ __device__ __forceinline__ void put_tile(float* A, f32x4 acc, const ChunkGates& 
 
 constexpr int MAX_TILES = 3;  // score tiles per wave (ten tiles over at least four waves)
 
-// LDS: K [CH][ks] | (delta) A [CH][AS] | inverted blocks | gate arrays
-template <typename TQ, typename TV, bool DELTA>
-__global__ __launch_bounds__(512) void memory_chunk_local_kernel(MemArgs a) {
+// NKK > 0: the keys fill up to 16 * NKK channels, known at compile time (0: any width).
+// LDS: K [CH][ks] | (delta) A [CH][AS] | inverted blocks | gate arrays.  A wave takes up to two column tiles, one after the other:
+// the value columns first, then (delta) the columns of the transition matrix.
+template <typename TQ, typename TV, bool DELTA, int NKK>
+__global__ __launch_bounds__(512, 4) void memory_chunk_local_kernel(MemArgs a) {
   extern __shared__ __attribute__((aligned(16))) float smem[];
   const int p = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6;
   const int t0 = a.cu[p], n = a.cu[p + 1] - t0;
-  const int dk = a.dk, dv = a.dv, dkp = (dk + 15) & ~15, ks = dkp + 4, nkk = dkp / 16;
+  const int dk = a.dk, dv = a.dv, dkt = (dk + 15) & ~15, nkk = NKK > 0 ? NKK : dkt / 16, dkp = 16 * nkk, ks = dkp + 4;
   float* Ks = smem;
   float* A = Ks + CH * ks;
   float* Tb = A + (DELTA ? CH * AS : 0);
   float* gl = Tb + (DELTA ? 4 * 16 * TBS : 0);
   const ChunkGates cg{gl, gl + CH, gl + 2 * CH, gl + 3 * CH, gl + 4 * CH};
-  const int nvt = ((dv + 15) / 16 + nw - 1) / nw;
-  const bool carry = DELTA && (int)blockIdx.z >= nvt;  // columns of the transition matrix
-  const int ct = (carry ? (int)blockIdx.z - nvt : (int)blockIdx.z) * nw + wave;
-  const int col = ct * 16 + (lane & 15), g4 = (lane >> 4) * 4;
-  const bool live = ct * 16 < (carry ? dk : dv);
+  const int vtiles = (dv + 15) / 16, tiles = vtiles + (DELTA ? dkt / 16 : 0);
+  const int g4 = (lane >> 4) * 4;
   const TQ* kp = reinterpret_cast<const TQ*>(a.k) + t0 * a.k_st + (h / a.rep) * a.k_sh;
   const TV* vp = reinterpret_cast<const TV*>(a.v) + t0 * a.v_st + h * a.v_sh;
+  const RawGates raw = load_gates<TV>(a, h, t0, n);
   f32x4 y[4];
+  auto load_values = [&](int ct) {
+    const int col = ct * 16 + (lane & 15);
 #pragma unroll
-  for (int m = 0; m < 4; ++m)
+    for (int m = 0; m < 4; ++m)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = 16 * m + g4 + r;
-      y[m][r] = (!carry && col < dv && t < n) ? ldf(vp + t * a.v_st + col) : 0.f;
-    }
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * m + g4 + r;
+        y[m][r] = (ct < vtiles && col < dv && t < n) ? ldf(vp + t * a.v_st + col) : 0.f;
+      }
+  };
+  int ct = (int)blockIdx.z * 2 * nw + wave;
+  load_values(ct);
   stage_rows(Ks, ks, kp, a.k_st, n, dk, dkp, a.vec != 0);
-  chunk_gates<TV>(a, cg, h, t0, n);
+  chunk_gates(a, cg, raw, h, n);
   __syncthreads();
   if constexpr (DELTA) {
     for (int i = wave; i < 10; i += nw) {
       int ti, tj;
       lower_tile(i, ti, tj);
-      put_tile(A, score_tile(Ks, Ks, ks, nkk, ti, tj, lane), cg, ti, tj, lane, true, cg.beta, nullptr);
+      put_tile(A, score_tile<NKK>(Ks, Ks, ks, nkk, ti, tj, lane), cg, ti, tj, lane, true, cg.beta, nullptr);
     }
     __syncthreads();
     invert_diagonals(A, Tb);
     __syncthreads();
   }
-  if (blockIdx.z == 0 && tid == 0 && a.dec != nullptr) a.dec[(int64_t)p * a.H + h] = cg.grow[CH - 1];
-  if (!live) return;
-#pragma unroll
-  for (int m = 0; m < 4; ++m)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = 16 * m + g4 + r;
-      if (carry) y[m][r] = -cg.grow[t] * Ks[t * ks + col];  // (dkp columns are staged)
-      y[m][r] *= cg.beta[t];
-    }
-  if constexpr (DELTA) solve(A, Tb, y, lane);
-#pragma unroll
-  for (int m = 0; m < 4; ++m)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) y[m][r] *= cg.rest[16 * m + g4 + r];
-  const float all = cg.grow[CH - 1];
-  for (int dt = 0; dt < nkk; ++dt) {
-    f32x4 acc;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) acc[r] = (carry && 16 * dt + g4 + r == col) ? all : 0.f;
+  if (blockIdx.z == 0 && tid == 0) a.dec[(int64_t)p * a.H + h] = cg.grow[CH - 1];
+#pragma unroll 1
+  for (int half = 0; half < 2; ++half, ct += nw) {
+    if (ct >= tiles) return;
+    asm volatile("" ::: "memory");  // the second tile reads LDS again: kept in registers over the loop, it would spill
+    if (half > 0) load_values(ct);
+    const bool carry = DELTA && ct >= vtiles;  // columns of the transition matrix
+    const int col = (carry ? ct - vtiles : ct) * 16 + (lane & 15);
 #pragma unroll
     for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) acc = mfma4(Ks[(16 * m + g4 + j) * ks + 16 * dt + (lane & 15)], y[m][j], acc);
-    if (carry) {
-      float* o = a.trans + (((int64_t)p * a.H + h) * dkp + 16 * dt + g4) * dkp + col;
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * m + g4 + r;
+        if (carry) y[m][r] = -cg.grow[t] * Ks[t * ks + col];
+        y[m][r] *= cg.beta[t];
+      }
+    if constexpr (DELTA) solve(A, Tb, y, lane);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) o[r * dkp] = acc[r];
-    } else if (col < dv) {
-      float* o = a.loc + (((int64_t)p * a.H + h) * dk + 16 * dt + g4) * dv + col;
+    for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int r = 0; r < 4; ++r)
-        if (16 * dt + g4 + r < dk) o[(int64_t)r * dv] = acc[r];
+      for (int r = 0; r < 4; ++r) y[m][r] *= cg.rest[16 * m + g4 + r];
+    const float all = cg.grow[CH - 1];
+    for (int dt = 0; dt < dkt / 16; ++dt) {
+      f32x4 acc;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) acc[r] = (carry && 16 * dt + g4 + r == col) ? all : 0.f;
+#pragma unroll
+      for (int m = 0; m < 4; ++m)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc = mfma4(Ks[(16 * m + g4 + j) * ks + 16 * dt + (lane & 15)], y[m][j], acc);
+      if (carry) {
+        float* o = a.trans + (((int64_t)p * a.H + h) * dkt + 16 * dt + g4) * dkt + col;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[r * dkt] = acc[r];
+      } else if (col < dv) {
+        float* o = a.loc + (((int64_t)p * a.H + h) * dk + 16 * dt + g4) * dv + col;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (16 * dt + g4 + r < dk) o[(int64_t)r * dv] = acc[r];
+      }
     }
   }
 }
 
 // LDS: K [CH][ks] | Q [CH][ks], later the read-out scores [CH][AS] | (delta) A [CH][AS] | inverted blocks | gate arrays
-template <typename TQ, typename TV, bool DELTA>
-__global__ __launch_bounds__(512) void memory_chunks_kernel(MemArgs a) {
+template <typename TQ, typename TV, bool DELTA, int NKK>
+__global__ __launch_bounds__(512, NKK == 8 && DELTA ? 2 : 4) void memory_chunks_kernel(MemArgs a) {
   extern __shared__ __attribute__((aligned(16))) float smem[];
   const int p = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6;
   const int t0 = a.cu[p], n = a.cu[p + 1] - t0;
   if (n <= 0) return;
-  const int dk = a.dk, dv = a.dv, dkp = (dk + 15) & ~15, ks = dkp + 4, nkk = dkp / 16;
+  const int dk = a.dk, dv = a.dv, nkk = NKK > 0 ? NKK : (dk + 15) / 16, dkp = 16 * nkk, ks = dkp + 4;
   float* Ks = smem;
   float* Qs = Ks + CH * ks;
   float* A = Qs + CH * (ks > AS ? ks : AS);
@@ -385,6 +463,7 @@ __global__ __launch_bounds__(512) void memory_chunks_kernel(MemArgs a) {
   const TV* vp = reinterpret_cast<const TV*>(a.v) + t0 * a.v_st + h * a.v_sh;
   const bool fresh = whole && a.start[p] == 0;
   const float* S0 = (whole ? a.S + ((int64_t)a.slots[p] * a.H + h) * dk * dv : a.init + ((int64_t)p * a.H + h) * dk * dv) + colc;
+  const RawGates raw = load_gates<TV>(a, h, t0, n);
   f32x4 y[4];
 #pragma unroll
   for (int m = 0; m < 4; ++m)
@@ -393,9 +472,36 @@ __global__ __launch_bounds__(512) void memory_chunks_kernel(MemArgs a) {
       const int t = 16 * m + g4 + r;
       y[m][r] = (cok && t < n) ? ldf(vp + t * a.v_st + col) : 0.f;
     }
+  // this wave's columns of the memory, requested ahead of everything that does not need them
+  f32x4 s0[NKK > 0 ? NKK : 1];
+  auto load_memory = [&](int kk) {
+    f32x4 s;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int d = 16 * kk + g4 + j;
+      s[j] = (live && !fresh && d < dk) ? S0[(int64_t)d * dv] : 0.f;
+    }
+    return s;
+  };
+  if constexpr (NKK > 0) {
+#pragma unroll
+    for (int kk = 0; kk < NKK; ++kk) s0[kk] = load_memory(kk);
+  }
   stage_rows(Ks, ks, kp, a.k_st, n, dk, dkp, a.vec != 0);
   stage_rows(Qs, ks, qp, a.q_st, n, dk, dkp, a.vec != 0);
-  chunk_gates<TV>(a, cg, h, t0, n);
+  const bool fused = a.y != nullptr;  // (one column tile per wave covers the head)
+  f32x4 gt[4];
+  auto load_gate = [&]() {
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * m + g4 + r;
+        gt[m][r] = (fused && cok && t < n) ? ldf(reinterpret_cast<const TV*>(a.hn_g) + (t0 + t) * a.hn_st + h * dv + col) : 0.f;
+      }
+  };
+  if constexpr (NKK != 8) load_gate();  // (the widest form has no registers to spare for it)
+  chunk_gates(a, cg, raw, h, n);
   __syncthreads();
   // scores of this wave's tiles (kept in registers: they overwrite Q), and this wave's columns of Q S_0 and K S_0
   f32x4 sq[MAX_TILES];
@@ -405,8 +511,8 @@ __global__ __launch_bounds__(512) void memory_chunks_kernel(MemArgs a) {
     if (tile < 10) {
       int ti, tj;
       lower_tile(tile, ti, tj);
-      sq[i] = score_tile(Qs, Ks, ks, nkk, ti, tj, lane);
-      if constexpr (DELTA) put_tile(A, score_tile(Ks, Ks, ks, nkk, ti, tj, lane), cg, ti, tj, lane, true, cg.beta, nullptr);
+      sq[i] = score_tile<NKK>(Qs, Ks, ks, nkk, ti, tj, lane);
+      if constexpr (DELTA) put_tile(A, score_tile<NKK>(Ks, Ks, ks, nkk, ti, tj, lane), cg, ti, tj, lane, true, cg.beta, nullptr);
     }
   }
   f32x4 oq[4], ok[4];
@@ -416,18 +522,18 @@ __global__ __launch_bounds__(512) void memory_chunks_kernel(MemArgs a) {
     for (int r = 0; r < 4; ++r) oq[m][r] = 0.f, ok[m][r] = 0.f;
   if (live && !fresh) {
     const int row = (lane & 15) * ks + g4;
-    for (int kk = 0; kk < nkk; ++kk) {
-      f32x4 s;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int d = 16 * kk + g4 + j;
-        s[j] = d < dk ? S0[(int64_t)d * dv] : 0.f;
-      }
+    auto read_out = [&](int kk, f32x4 s) {
 #pragma unroll
       for (int m = 0; m < 4; ++m) {
         oq[m] = block_product(lds4(Qs + 16 * m * ks + row + 16 * kk), s, oq[m]);
         if constexpr (DELTA) ok[m] = block_product(lds4(Ks + 16 * m * ks + row + 16 * kk), s, ok[m]);
       }
+    };
+    if constexpr (NKK > 0) {
+#pragma unroll
+      for (int kk = 0; kk < NKK; ++kk) read_out(kk, s0[kk]);
+    } else {
+      for (int kk = 0; kk < nkk; ++kk) read_out(kk, load_memory(kk));
     }
   }
   __syncthreads();
@@ -442,7 +548,7 @@ __global__ __launch_bounds__(512) void memory_chunks_kernel(MemArgs a) {
   }
   if constexpr (DELTA) invert_diagonals(A, Tb);
   __syncthreads();
-  if (!live) return;
+  if (!live && !fused) return;
   const float sk = a.skip != nullptr ? a.skip[h] : 0.f;
   if constexpr (DELTA) {
 #pragma unroll
@@ -461,11 +567,44 @@ __global__ __launch_bounds__(512) void memory_chunks_kernel(MemArgs a) {
     for (int r = 0; r < 4; ++r) o[r] = cg.grow[16 * m + g4 + r] * oq[m][r] + (DELTA ? 0.f : sk * y[m][r]);
 #pragma unroll
     for (int c = 0; c <= m; ++c) o = block_product(lds4(Qs + (16 * m + (lane & 15)) * AS + 16 * c + g4), y[c], o);
+    oq[m] = o;
+  }
+  if (fused) {
+    float* rstd = gl + 5 * CH;
+    float* part = rstd + CH;  // [waves][CH] sums of squares of a wave's columns
+    if constexpr (NKK == 8) load_gate();
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = 16 * m + g4 + r;
-      if (cok && t < n) a.out[((int64_t)(t0 + t) * a.H + h) * dv + col] = o[r];
+    for (int m = 0; m < 4; ++m) {
+      f32x4 q;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) q[r] = sum16(cok ? oq[m][r] * oq[m][r] : 0.f);
+      if ((lane & 15) == 0) *reinterpret_cast<f32x4*>(part + wave * CH + 16 * m + g4) = q;
     }
+    __syncthreads();
+    if (tid < CH) {
+      float q = 0.f;
+      for (int x = 0; x < nw; ++x) q += part[x * CH + tid];
+      rstd[tid] = 1.0f / sqrtf(q / (float)dv + a.hn_eps);
+    }
+    __syncthreads();
+    const float w = (a.hn_w != nullptr && cok) ? a.hn_w[h * dv + col] : 1.f;
+    TV* yp = reinterpret_cast<TV*>(a.y) + ((int64_t)t0 * a.H + h) * dv + col;
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * m + g4 + r;
+        if (cok && t < n) stf(yp + (int64_t)t * a.H * dv, oq[m][r] * rstd[t] * w * silu(gt[m][r]));
+      }
+    if (!live) return;
+  } else {
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * m + g4 + r;
+        if (cok && t < n) a.out[((int64_t)(t0 + t) * a.H + h) * dv + col] = oq[m][r];
+      }
   }
   if (!whole) return;
 #pragma unroll
@@ -646,9 +785,21 @@ void set_pool(MemArgs& a, const at::Tensor& S) {
   a.S = S.data_ptr<float>();
 }
 
-void set_out(MemArgs& a, const at::Tensor& out, int64_t T) {
-  HYB_CHECK(f32vec(out, T * a.H * a.dv), "out: fp32 [T, H, dv]");
-  a.out = out.data_ptr<float>();
+// the outputs: fp32 [T, H, dv], or (a gate given) the head norm's result [T, H * dv] in v's dtype
+void set_out(MemArgs& a, const at::Tensor& out, const at::Tensor& v, const OptT& hn_w, const OptT& hn_g, double eps) {
+  const int64_t T = v.size(0), n = a.H * (int64_t)a.dv;
+  if (!hn_g.has_value()) {
+    HYB_CHECK(f32vec(out, T * n) && !hn_w.has_value(), "out: fp32 [T, H, dv]");
+    a.out = out.data_ptr<float>();
+    return;
+  }
+  HYB_CHECK(a.dv % 4 == 0 && a.dv <= 128, "the fused head norm takes value sizes up to 128 in quads");
+  HYB_CHECK(out.is_cuda() && out.is_contiguous() && out.scalar_type() == v.scalar_type() && out.numel() == T * n, "out: [T, H * dv] of v's dtype");
+  check_rows(*hn_g, "gate");
+  HYB_CHECK(hn_g->size(0) == T && hn_g->size(1) == n && hn_g->scalar_type() == v.scalar_type(), "gate: [T, H * dv] of v's dtype");
+  HYB_CHECK(!hn_w.has_value() || f32vec(*hn_w, n), "norm weight: fp32 [H * dv]");
+  a.y = out.data_ptr(), a.hn_g = hn_g->data_ptr(), a.hn_st = hn_g->stride(0), a.hn_eps = (float)eps;
+  a.hn_w = hn_w.has_value() ? hn_w->data_ptr<float>() : nullptr;
 }
 
 // q / k dtype x v dtype: (v, v) or (fp32, v)
@@ -662,6 +813,16 @@ void dispatch_qv(const at::Tensor& q, const at::Tensor& v, F&& f) {
 
 int waves_for(int dv) { return dv > 64 ? 8 : 4; }
 
+// channels that a chunk's keys take in LDS: the compile-time widths 32, 64 and 128, else filled up to 16
+int staged_width(int dk) { return dk <= 32 ? 32 : (dk <= 64 ? 64 : (dk <= 128 && dk > 96 ? 128 : (dk + 15) / 16 * 16)); }
+template <typename F>
+void by_width(int dk, F&& f) {
+  if (dk <= 32) f(std::integral_constant<int, 2>());
+  else if (dk <= 64) f(std::integral_constant<int, 4>());
+  else if (dk <= 128 && dk > 96) f(std::integral_constant<int, 8>());
+  else f(std::integral_constant<int, 0>());
+}
+
 template <typename K>
 void launch_lds(K kern, dim3 grid, int threads, size_t lds, const MemArgs& a) {
   HYB_CHECK(lds <= 160 * 1024, "keys too wide for LDS");
@@ -673,32 +834,33 @@ void launch_lds(K kern, dim3 grid, int threads, size_t lds, const MemArgs& a) {
 
 void memory_decode(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, int64_t kind, const OptT& ga, const OptT& gb, const OptT& a_log,
                    const OptT& dt_bias, const OptT& log_decay, const OptT& skip, at::Tensor S, const at::Tensor& slots, const at::Tensor& start,
-                   at::Tensor out, int64_t row0) {
+                   at::Tensor out, const OptT& hn_w, const OptT& hn_g, double hn_eps, int64_t row0) {
   MemArgs a = mem_args(q, k, v, kind, ga, gb, a_log, dt_bias, log_decay, skip);
   set_pool(a, S);
-  set_out(a, out, v.size(0));
+  set_out(a, out, v, hn_w, hn_g, hn_eps);
   HYB_CHECK(i32(slots) && i32(start) && slots.numel() == start.numel() && row0 >= 0 && row0 + slots.numel() == v.size(0), "slots [n], start [n]: the last n rows");
   const int64_t n = slots.numel();
   if (n == 0) return;
   a.slots = slots.data_ptr<int>(), a.start = start.data_ptr<int>(), a.row0 = (int)row0;
   c10::DeviceGuard guard(v.device());
-  const bool v4 = a.dv % 4 == 0;
-  const int tile = v4 ? 64 : 16;
+  const bool v4 = a.dv % 4 == 0, wide = v4 && a.dv > 64 && a.dv <= 128;  // (a head of up to 128 values is one tile)
+  const int tile = wide ? 128 : (v4 ? 64 : 16);
   const dim3 grid((unsigned)n, (unsigned)a.H, (unsigned)((a.dv + tile - 1) / tile));
   dispatch_qv(q, v, [&](auto* tq, auto* tv) {
     using TQ = std::remove_pointer_t<decltype(tq)>;
     using TV = std::remove_pointer_t<decltype(tv)>;
-    auto go = [&](auto kern) { kern<<<grid, 256, 0, cur_stream()>>>(a); };
-    auto rows = [&](auto vec) {
-      constexpr int V = decltype(vec)::value;
-      if (a.dk <= 16) go(memory_decode_kernel<TQ, TV, V, 1>);
-      else if (a.dk <= 32) go(memory_decode_kernel<TQ, TV, V, 2>);
-      else if (a.dk <= 64) go(memory_decode_kernel<TQ, TV, V, 4>);
-      else if (a.dk <= 128) go(memory_decode_kernel<TQ, TV, V, 8>);
-      else go(memory_decode_kernel<TQ, TV, V, 16>);
+    auto go = [&](auto kern, int cl) { kern<<<grid, 16 * cl, 0, cur_stream()>>>(a); };
+    auto rows = [&](auto vec, auto lanes) {
+      constexpr int V = decltype(vec)::value, CL = decltype(lanes)::value;
+      if (a.dk <= 16) go(memory_decode_kernel<TQ, TV, V, 1, CL>, CL);
+      else if (a.dk <= 32) go(memory_decode_kernel<TQ, TV, V, 2, CL>, CL);
+      else if (a.dk <= 64) go(memory_decode_kernel<TQ, TV, V, 4, CL>, CL);
+      else if (a.dk <= 128) go(memory_decode_kernel<TQ, TV, V, 8, CL>, CL);
+      else go(memory_decode_kernel<TQ, TV, V, 16, CL>, CL);
     };
-    if (v4) rows(std::integral_constant<int, 4>());
-    else rows(std::integral_constant<int, 1>());
+    if (wide) rows(std::integral_constant<int, 4>(), std::integral_constant<int, 32>());
+    else if (v4) rows(std::integral_constant<int, 4>(), std::integral_constant<int, 16>());
+    else rows(std::integral_constant<int, 1>(), std::integral_constant<int, 16>());
   });
 }
 
@@ -706,10 +868,10 @@ void memory_decode(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v
 // of longer ones and start from init
 void memory_chunks(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, int64_t kind, const OptT& ga, const OptT& gb, const OptT& a_log,
                    const OptT& dt_bias, const OptT& log_decay, const OptT& skip, at::Tensor S, const OptT& slots, const at::Tensor& cu,
-                   const OptT& start, const OptT& init, at::Tensor out, int64_t rows) {
+                   const OptT& start, const OptT& init, at::Tensor out, const OptT& hn_w, const OptT& hn_g, double hn_eps, int64_t rows) {
   MemArgs a = mem_args(q, k, v, kind, ga, gb, a_log, dt_bias, log_decay, skip);
   set_pool(a, S);
-  set_out(a, out, v.size(0));
+  set_out(a, out, v, hn_w, hn_g, hn_eps);
   HYB_CHECK(i32(cu) && cu.numel() >= 1 && rows >= 0 && rows <= v.size(0), "cu: int32 [n + 1]");
   const int64_t n = cu.numel() - 1;
   if (n == 0 || rows == 0) return;
@@ -722,15 +884,19 @@ void memory_chunks(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v
     a.slots = slots->data_ptr<int>(), a.start = start->data_ptr<int>();
   }
   c10::DeviceGuard guard(v.device());
-  const int nw = waves_for(a.dv), dkp = (a.dk + 15) / 16 * 16, ks = dkp + 4;
+  const int nw = waves_for(a.dv), ks = staged_width(a.dk) + 4;
   const bool delta = kind == KIND_DELTA;
-  const size_t lds = sizeof(float) * (size_t)(CH * ks + CH * std::max(ks, AS) + (delta ? CH * AS + 4 * 16 * TBS : 0) + 5 * CH);
+  const size_t lds = sizeof(float) * (size_t)(CH * ks + CH * std::max(ks, AS) + (delta ? CH * AS + 4 * 16 * TBS : 0) + 5 * CH + (a.y != nullptr ? (nw + 1) * CH : 0));
   const dim3 grid((unsigned)n, (unsigned)a.H, (unsigned)(((a.dv + 15) / 16 + nw - 1) / nw));
   dispatch_qv(q, v, [&](auto* tq, auto* tv) {
     using TQ = std::remove_pointer_t<decltype(tq)>;
     using TV = std::remove_pointer_t<decltype(tv)>;
-    if (delta) launch_lds(memory_chunks_kernel<TQ, TV, true>, grid, 64 * nw, lds, a);
-    else launch_lds(memory_chunks_kernel<TQ, TV, false>, grid, 64 * nw, lds, a);
+    auto go = [&](auto nkk) {
+      constexpr int N = decltype(nkk)::value;
+      if (delta) launch_lds(memory_chunks_kernel<TQ, TV, true, N>, grid, 64 * nw, lds, a);
+      else launch_lds(memory_chunks_kernel<TQ, TV, false, N>, grid, 64 * nw, lds, a);
+    };
+    by_width(a.dk, go);
   });
 }
 
@@ -741,7 +907,7 @@ void memory_chunk_local(const at::Tensor& q, const at::Tensor& k, const at::Tens
   HYB_CHECK(i32(cu) && cu.numel() >= 1, "cu: int32 [chunks + 1]");
   const int64_t n = cu.numel() - 1;
   if (n == 0) return;
-  const int nw = waves_for(a.dv), dkp = (a.dk + 15) / 16 * 16, ks = dkp + 4;
+  const int nw = waves_for(a.dv), dkp = (a.dk + 15) / 16 * 16, ks = staged_width(a.dk) + 4;
   const bool delta = kind == KIND_DELTA;
   HYB_CHECK(f32vec(loc, n * a.H * a.dk * a.dv) && f32vec(dec, n * a.H), "loc: fp32 [chunks, H, dk, dv], dec: fp32 [chunks, H]");
   HYB_CHECK(trans.has_value() == delta && (!delta || f32vec(*trans, n * a.H * dkp * dkp)), "trans: fp32 [chunks, H, dkp, dkp] (delta kind), dkp = dk filled up to 16");
@@ -749,13 +915,17 @@ void memory_chunk_local(const at::Tensor& q, const at::Tensor& k, const at::Tens
   a.trans = delta ? trans->data_ptr<float>() : nullptr;
   c10::DeviceGuard guard(v.device());
   const size_t lds = sizeof(float) * (size_t)(CH * ks + (delta ? CH * AS + 4 * 16 * TBS : 0) + 5 * CH);
-  const int tiles = ((a.dv + 15) / 16 + nw - 1) / nw + (delta ? (dkp / 16 + nw - 1) / nw : 0);
-  const dim3 grid((unsigned)n, (unsigned)a.H, (unsigned)tiles);
+  const int tiles = (a.dv + 15) / 16 + (delta ? dkp / 16 : 0);
+  const dim3 grid((unsigned)n, (unsigned)a.H, (unsigned)((tiles + 2 * nw - 1) / (2 * nw)));
   dispatch_qv(q, v, [&](auto* tq, auto* tv) {
     using TQ = std::remove_pointer_t<decltype(tq)>;
     using TV = std::remove_pointer_t<decltype(tv)>;
-    if (delta) launch_lds(memory_chunk_local_kernel<TQ, TV, true>, grid, 64 * nw, lds, a);
-    else launch_lds(memory_chunk_local_kernel<TQ, TV, false>, grid, 64 * nw, lds, a);
+    auto go = [&](auto nkk) {
+      constexpr int N = decltype(nkk)::value;
+      if (delta) launch_lds(memory_chunk_local_kernel<TQ, TV, true, N>, grid, 64 * nw, lds, a);
+      else launch_lds(memory_chunk_local_kernel<TQ, TV, false, N>, grid, 64 * nw, lds, a);
+    };
+    by_width(a.dk, go);
   });
 }
 

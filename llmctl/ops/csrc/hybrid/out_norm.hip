@@ -47,15 +47,16 @@ bool rows4(const at::Tensor& t) {  // rows that 4-element accesses may walk
   return t.stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(t.data_ptr()) % (4 * sizeof(T)) == 0;
 }
 
-template <typename T>
+template <typename T, int N>
 __global__ __launch_bounds__(NT) void embed_f32_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table, float* __restrict__ x,
                                                        T* __restrict__ h, int W) {
   const int64_t row = blockIdx.x;
   const T* e = table + ids[row] * (int64_t)W;
-  for (int c = threadIdx.x; c < W; c += NT) {
-    const T v = e[c];
-    h[row * W + c] = v;
-    x[row * W + c] = ldf(&v);
+  for (int c = threadIdx.x * N; c < W; c += NT * N) {
+    float v[N];
+    ldn<T, N>(e + c, v);
+    stn<T, N>(h + row * W + c, v);
+    stn<float, N>(x + row * W + c, v);
   }
 }
 
@@ -234,8 +235,11 @@ std::tuple<at::Tensor, at::Tensor> embed_f32(const at::Tensor& ids, const at::Te
   if (T == 0) return {x, h};
   dispatch_act(table, [&](auto* tag) {
     using Tt = std::remove_pointer_t<decltype(tag)>;
-    embed_f32_kernel<Tt><<<dim3((unsigned)T), NT, 0, cur_stream()>>>(ids.data_ptr<int64_t>(), (const Tt*)table.data_ptr(), x.data_ptr<float>(),
-                                                                   (Tt*)h.data_ptr(), (int)W);
+    auto go = [&](auto kern) {
+      kern<<<dim3((unsigned)T), NT, 0, cur_stream()>>>(ids.data_ptr<int64_t>(), (const Tt*)table.data_ptr(), x.data_ptr<float>(), (Tt*)h.data_ptr(), (int)W);
+    };
+    if (W % 4 == 0 && rows4<Tt>(table)) go(embed_f32_kernel<Tt, 4>);
+    else go(embed_f32_kernel<Tt, 1>);
   });
   return {x, h};
 }

@@ -175,6 +175,50 @@ __global__ __launch_bounds__(NT) void headnorm_gate_kernel(const float* __restri
   }
 }
 
+// The same for heads of at most 256 values in quads: ``lg`` lanes (a power of two) own a head, four neighbouring entries each.
+template <typename T>
+__global__ __launch_bounds__(NT) void headnorm_gate_quads_kernel(const float* __restrict__ o, const float* __restrict__ w,
+                                                                 const T* __restrict__ g, int64_t g_stride, T* __restrict__ y,
+                                                                 int64_t pairs, int H, int dv, float eps, int silu, int lg) {
+  const int64_t p = ((int64_t)blockIdx.x * NT + threadIdx.x) / lg;
+  if (p >= pairs) return;  // (a head's lanes leave together)
+  const int c = (threadIdx.x % lg) * 4;
+  const bool ok = c < dv;
+  const int64_t t = p / H;
+  const int hd = (int)(p - t * H);
+  float v[4] = {0.f, 0.f, 0.f, 0.f}, gv[4] = {0.f, 0.f, 0.f, 0.f}, wv[4] = {1.f, 1.f, 1.f, 1.f};
+  if (ok) {
+    Vec16<float>::load(o + p * dv + c, v);
+    const T* gp = g + t * g_stride + hd * dv + c;
+    if constexpr (sizeof(T) == 4) {
+      Vec16<float>::load(reinterpret_cast<const float*>(gp), gv);
+    } else {
+      const uint2 x = *reinterpret_cast<const uint2*>(gp);
+      gv[0] = __uint_as_float(x.x << 16), gv[1] = __uint_as_float(x.x & 0xffff0000u);
+      gv[2] = __uint_as_float(x.y << 16), gv[3] = __uint_as_float(x.y & 0xffff0000u);
+    }
+    if (w != nullptr) Vec16<float>::load(w + hd * dv + c, wv);
+  }
+  float q = (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+  for (int s = lg >> 1; s > 0; s >>= 1) q += __shfl_xor(q, s, 64);
+  if (!ok) return;
+  const float rstd = 1.0f / sqrtf(q / (float)dv + eps);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const float gate = 1.0f / (1.0f + expf(-gv[i]));
+    v[i] *= rstd * wv[i] * (silu ? gv[i] * gate : gate);
+  }
+  if constexpr (sizeof(T) == 4) {
+    Vec16<float>::store(reinterpret_cast<float*>(y) + p * dv + c, v);
+  } else {
+    unsigned x[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      x[i] = (unsigned)__bfloat16_as_ushort(__float2bfloat16(v[2 * i])) | ((unsigned)__bfloat16_as_ushort(__float2bfloat16(v[2 * i + 1])) << 16);
+    *reinterpret_cast<uint2*>(y + p * dv + c) = make_uint2(x[0], x[1]);
+  }
+}
+
 // ------------------------------------------------------------------------------------------ host
 static at::Tensor out_like(const at::Tensor& ref, at::IntArrayRef shape, bool bf16) {
   return at::empty(shape, ref.options().dtype(bf16 ? at::kBFloat16 : at::kFloat));
@@ -349,6 +393,16 @@ at::Tensor headnorm_gate(const at::Tensor& o, const c10::optional<at::Tensor>& w
   const int64_t pairs = T * H;
   dispatch_act(g, [&](auto* tag) {
     using Tt = std::remove_pointer_t<decltype(tag)>;
+    const bool quads = dv % 4 == 0 && dv <= 256 && g.stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(g.data_ptr()) % (4 * sizeof(Tt)) == 0 &&
+                       reinterpret_cast<uintptr_t>(o.data_ptr()) % 16 == 0 && (!w.has_value() || reinterpret_cast<uintptr_t>(w->data_ptr()) % 16 == 0);
+    if (quads) {
+      int lg = 1;
+      while (lg * 4 < dv) lg *= 2;
+      headnorm_gate_quads_kernel<Tt><<<dim3((unsigned)((pairs * lg + NT - 1) / NT)), NT, 0, cur_stream()>>>(
+          o.data_ptr<float>(), w.has_value() ? w->data_ptr<float>() : nullptr, (const Tt*)g.data_ptr(), g.stride(0), (Tt*)y.data_ptr(), pairs, H, dv,
+          (float)eps, silu ? 1 : 0, lg);
+      return;
+    }
     headnorm_gate_kernel<Tt><<<dim3((unsigned)((pairs + NW - 1) / NW)), NT, 0, cur_stream()>>>(
         o.data_ptr<float>(), w.has_value() ? w->data_ptr<float>() : nullptr, (const Tt*)g.data_ptr(), g.stride(0), (Tt*)y.data_ptr(), pairs, H, dv, (float)eps, silu ? 1 : 0);
   });

@@ -604,7 +604,7 @@ def _memory_plan(b, device):
     return b.scratch["memory_plan"]
 
 
-def memory_scan(q, k, v, kind: str, S, b, ga=None, gb=None, a_log=None, dt_bias=None, log_decay=None, skip=None):
+def memory_scan(q, k, v, kind: str, S, b, ga=None, gb=None, a_log=None, dt_bias=None, log_decay=None, skip=None, norm=None):
     """A matrix memory per head with one decay per head and token, over the step's tokens: ``S <- g S``, ``S <- S + k u^T``,
     ``o = S^T q`` with ``u = beta v``, or ``u = beta (v - S^T k)`` (what the decayed memory gives for k is taken off first).
 
@@ -613,24 +613,33 @@ def memory_scan(q, k, v, kind: str, S, b, ga=None, gb=None, a_log=None, dt_bias=
     form of u.  ``q, k [T, KH, dk]`` (one dtype; head h of H reads h // (H / KH)), ``v [T, H, dv]`` (row-strided views
     allowed), ``ga, gb [T, H]`` in v's dtype, ``a_log, dt_bias, log_decay, skip`` fp32 ``[H]``; ``skip``: o gains ``skip_h v``.
     Returns fp32 ``[T, H, dv]`` and updates the state pool ``S`` (fp32 ``[slots, H, dk, dv]``) in place at ``b.state`` (a
-    sequence that starts at position 0 begins from zeros).
+    sequence that starts at position 0 begins from zeros).  ``norm`` = (weight fp32 ``[H*dv]`` or None, gate ``[T, H*dv]``, eps):
+    returns :func:`headnorm_gate` of the outputs with silu, ``[T, H*dv]`` in v's dtype (in the same kernels for value sizes
+    up to 128 in quads).
 
     Decode rows run one after the other in memory (a read and a write of S); prompt portions run in chunks of
     :data:`MEMORY_CHUNK` tokens whose products go to the fp32 matrix cores.  A portion of several chunks takes three
     passes: every chunk's own contribution (delta: and its transition product) at once, the memories at the
     chunks' first tokens in order, every chunk's outputs at once."""
     if not use_native(v):
-        return ref.memory_scan(q, k, v, kind, ga, gb, a_log, dt_bias, log_decay, skip, S, b.state, b.cu, b.start)
+        o = ref.memory_scan(q, k, v, kind, ga, gb, a_log, dt_bias, log_decay, skip, S, b.state, b.cu, b.start)
+        return o if norm is None else ref.headnorm_gate(o, norm[0], norm[1], norm[2], v.dtype, True)
     nat = native_hybrid()
     T, H, dv = v.shape
     dk = q.shape[2]
-    out = torch.empty(T, H, dv, device=v.device, dtype=torch.float32)
+    if norm is not None and (dv % 4 or dv > 128):
+        o = memory_scan(q, k, v, kind, S, b, ga, gb, a_log, dt_bias, log_decay, skip)
+        return headnorm_gate(o, *norm, v.dtype, True)
+    if norm is None:
+        out, ends = torch.empty(T, H, dv, device=v.device, dtype=torch.float32), (None, None, 0.0)
+    else:
+        out, ends = torch.empty(T, H * dv, device=v.device, dtype=v.dtype), norm
     gates = (MEMORY_KINDS[kind], ga, gb, a_log, dt_bias, log_decay, skip)
     if b.Tp:
         n = b.p_ctx.shape[0]
         plan = _memory_plan(b, v.device)
         if plan is None:
-            nat.memory_chunks(q, k, v, *gates, S, b.state[:n], b.cu[:n + 1], b.start[:n], None, out, b.Tp)
+            nat.memory_chunks(q, k, v, *gates, S, b.state[:n], b.cu[:n + 1], b.start[:n], None, out, *ends, b.Tp)
         else:
             pcu, base, P = plan
             f32 = dict(dtype=torch.float32, device=v.device)
@@ -641,10 +650,10 @@ def memory_scan(q, k, v, kind: str, S, b, ga=None, gb=None, a_log=None, dt_bias=
             init = torch.empty(P, H, dk, dv, **f32)
             nat.memory_chunk_local(q, k, v, *gates, pcu, loc, dec, trans)
             nat.memory_combine(S, b.state[:n], b.start[:n], base, loc, dec, trans, init)
-            nat.memory_chunks(q, k, v, *gates, S, None, pcu, None, init, out, b.Tp)
+            nat.memory_chunks(q, k, v, *gates, S, None, pcu, None, init, out, *ends, b.Tp)
     if T > b.Tp:
         n0 = b.cu.shape[0] - 1 - (T - b.Tp)
-        nat.memory_decode(q, k, v, *gates, S, b.state[n0:], b.start[n0:], out, b.Tp)
+        nat.memory_decode(q, k, v, *gates, S, b.state[n0:], b.start[n0:], out, *ends, b.Tp)
     return out
 
 

@@ -501,7 +501,7 @@ def memory_gates(kind, T, H, ga, gb, a_log, dt_bias, log_decay):
     """(log decay, write strength) fp32 [T, H] of :func:`memory_scan`."""
     if kind == "fixed":
         return log_decay.float()[None, :].expand(T, H), torch.ones(T, H)
-    dt = torch.nn.functional.softplus(ga.float() + dt_bias.float(), threshold=1e30)
+    dt = torch.nn.functional.softplus(ga.float() + dt_bias.float())
     la = -torch.exp(a_log.float()) * dt
     return la, (dt if kind == "ssm" else torch.sigmoid(gb.float()))
 

@@ -482,7 +482,15 @@ def _memory_case(dev, kind, steps, H, KH, dk, dv, seed, edit=None, qk32=None):
             kw["ga"] = ga.to(device)[:, 1:H + 1]
         if kind == "delta":
             kw["gb"] = gb.to(device)
+        gate, w = torch.randn(T, H * dv, generator=g).to(dtype), torch.randn(H * dv, generator=g)
+        eps = float((0.01 * want.abs().max()) ** 2)  # (rows far below the largest ones would show the fp32 rounding of those)
+        for weight in (None, w):  # the same with the head norm, on a copy of the memories
+            y = hybrid.memory_scan(wide(q), wide(k), wide(v), kind, pool.clone(), _batch(st, device), **kw,
+                                   norm=(weight.to(device) if weight is not None else None, wide(gate), eps))
+            ref = plain.rms(want, eps).reshape(T, -1) * plain.silu(gate.double()) * (weight.double() if weight is not None else 1.0)
+            assert y.dtype == dtype and float((y.double().cpu() - ref).abs().max() / ref.abs().max()) < (1e-3 if dtype == torch.float32 else 1e-2)
         got = hybrid.memory_scan(wide(q), wide(k), wide(v), kind, pool, _batch(st, device), **kw).double().cpu()
+        assert bool(torch.isfinite(got).all()) and bool(torch.isfinite(pool.cpu()).all())
         worst_o = max(worst_o, float((got - want).abs().max() / want.abs().max()))
         for _, _, s in st:
             worst_s = max(worst_s, float((pool[s].double().cpu() - state[s]).abs().max() / state[s].abs().max().clamp(min=1e-3)))
