@@ -198,15 +198,26 @@ struct ConvUnitArgs {
   const int* sslot;
   float* qk;  // [T, ng, dk]
   void* y;    // [T, C - ng * dk]
-  int T, C, taps, ng, nq, dk, lg, tok, whole;  // lg lanes per unit; tok tokens per walk, or (whole) a sequence per walk
+  int T, C, taps, ng, nq, dk, lg, whole;  // lg lanes per unit; whole: a sequence per walk
   float qscale, eps;
 };
 
-constexpr int CONV_WALK = 8;  // tokens per walk at most (CONV_SHORT fits)
-static_assert(CONV_SHORT <= CONV_WALK, "short portions are one walk");
+// the sum over a unit's ``lg`` lanes (a power of two), in each of them: inside a row of 16 by lane permutations, then across rows
+__device__ __forceinline__ float unit_sum(float v, int lg) {
+  auto add = [&](auto ctrl) { v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), decltype(ctrl)::value, 0xf, 0xf, true)); };
+  if (lg > 1) add(std::integral_constant<int, 0xB1>());   // neighbours of a pair
+  if (lg > 2) add(std::integral_constant<int, 0x4E>());   // pairs of a quad
+  if (lg > 4) add(std::integral_constant<int, 0x141>());  // quads of a half row
+  if (lg > 8) add(std::integral_constant<int, 0x140>());  // halves of a row
+  if (lg > 16) v += __shfl_xor(v, 16, 64);
+  if (lg > 32) v += __shfl_xor(v, 32, 64);
+  return v;
+}
 
-// A unit is a group of dk channels, or a span of lg * VEC * NI of the other channels.  TAPS == 0: any number of taps.
-template <typename T, int VEC, int NI, int TAPS>
+// A unit is a group of dk channels, or a span of lg * VEC * NI of the other channels.  TAPS == 0: any number of taps.  A walk of
+// WALK tokens that lies inside one sequence, its taps inside the step's rows, runs without branches on rows requested at
+// once; any other walk goes token by token.
+template <typename T, int VEC, int NI, int TAPS, int WALK>
 __global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
   constexpr int NH = TAPS > 1 ? TAPS - 1 : 1;
   const int lane = threadIdx.x % a.lg;
@@ -222,7 +233,7 @@ __global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
     t_lo = a.cu[blockIdx.x], t_hi = a.cu[blockIdx.x + 1];
     if (t_lo >= t_hi) return;
   } else {
-    t_lo = (int)blockIdx.x * a.tok, t_hi = min(t_lo + a.tok, a.T);
+    t_lo = (int)blockIdx.x * WALK, t_hi = min(t_lo + WALK, a.T);
   }
   const T* u = reinterpret_cast<const T*>(a.u);
   int ch[NI];
@@ -248,99 +259,20 @@ __global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
     if constexpr (VEC == 4) Vec16<float>::load(p, v);
     else v[0] = p[0];
   };
-  // the input ``k`` positions before token t of the sequence that begins at row s0, position p0
-  auto past = [&](int t, int k, int s0, int p0, const float* st, int i, float* v) {
-    const int j = t - s0 - k;
-    if (j >= 0) {
-      load_row(u + (int64_t)(t - k) * a.u_st + ch[i], v);
-    } else if (p0 + j >= 0) {
-      load_f(st + (int64_t)(taps - 1 + j) * a.C + ch[i], v);
-    } else {
+  // silu in place, then the unit's result for token t
+  auto activate = [&](float (&x)[NI][VEC]) {
+    float ss = 0.f;
 #pragma unroll
-      for (int c = 0; c < VEC; ++c) v[c] = 0.f;
-    }
-  };
-  float wk[TAPS > 0 ? TAPS : 1][NI][VEC], bs[NI][VEC];
-#pragma unroll
-  for (int i = 0; i < NI; ++i) {
-#pragma unroll
-    for (int c = 0; c < VEC; ++c) bs[i][c] = 0.f;
-    if (a.bias != nullptr) load_f(a.bias + ch[i], bs[i]);
-    if constexpr (TAPS > 0) {
-#pragma unroll
-      for (int k = 0; k < TAPS; ++k) load_f(a.w + (int64_t)k * a.C + ch[i], wk[k][i]);
-    }
-  }
-  float hist[NH][NI][VEC];  // hist[k]: the input k + 1 positions before the current token
-  float in[CONV_WALK][NI][VEC];  // the walk's inputs, requested at once
-#pragma unroll
-  for (int j = 0; j < CONV_WALK; ++j)
-    if (t_lo + j < t_hi) {
-#pragma unroll
-      for (int i = 0; i < NI; ++i) load_row(u + (int64_t)(t_lo + j) * a.u_st + ch[i], in[j][i]);
-    }
-  int s = a.whole ? (int)blockIdx.x : a.seq_of[t_lo];
-  int s0 = a.cu[s], s1 = a.cu[s + 1], p0 = a.start[s];
-  float* st = a.state + (int64_t)a.sslot[s] * (taps - 1) * a.C;
-#pragma unroll
-  for (int jt = 0; jt < CONV_WALK; ++jt) {
-    const int t = t_lo + jt;
-    if (t >= t_hi) break;
-    bool reload = jt == 0;
-    if (t >= s1) {
-      s = a.seq_of[t];
-      s0 = a.cu[s], s1 = a.cu[s + 1], p0 = a.start[s];
-      st = a.state + (int64_t)a.sslot[s] * (taps - 1) * a.C;
-      reload = true;
-    }
-    if constexpr (TAPS > 1) {
-      if (reload) {
-#pragma unroll
-        for (int k = 0; k < TAPS - 1; ++k)
-#pragma unroll
-          for (int i = 0; i < NI; ++i) past(t, k + 1, s0, p0, st, i, hist[k][i]);
-      }
-    }
-    float x[NI][VEC], ss = 0.f;
-#pragma unroll
-    for (int i = 0; i < NI; ++i) {
-      const float(&cur)[VEC] = in[jt][i];
-      if constexpr (TAPS > 0) {
-#pragma unroll
-        for (int c = 0; c < VEC; ++c) {
-          float acc = bs[i][c] + wk[TAPS - 1][i][c] * cur[c];
-#pragma unroll
-          for (int k = 0; k < TAPS - 1; ++k) acc += wk[TAPS - 2 - k][i][c] * hist[k][i][c];
-          x[i][c] = acc;
-        }
-#pragma unroll
-        for (int k = TAPS - 2; k > 0; --k)
-#pragma unroll
-          for (int c = 0; c < VEC; ++c) hist[k][i][c] = hist[k - 1][i][c];
-        if constexpr (TAPS > 1) {
-#pragma unroll
-          for (int c = 0; c < VEC; ++c) hist[0][i][c] = cur[c];
-        }
-      } else {
-        float w1[VEC], v[VEC];
-        load_f(a.w + (int64_t)(taps - 1) * a.C + ch[i], w1);
-#pragma unroll
-        for (int c = 0; c < VEC; ++c) x[i][c] = bs[i][c] + w1[c] * cur[c];
-        for (int k = 1; k < taps; ++k) {
-          past(t, k, s0, p0, st, i, v);
-          load_f(a.w + (int64_t)(taps - 1 - k) * a.C + ch[i], w1);
-#pragma unroll
-          for (int c = 0; c < VEC; ++c) x[i][c] += w1[c] * v[c];
-        }
-      }
+    for (int i = 0; i < NI; ++i)
 #pragma unroll
       for (int c = 0; c < VEC; ++c) {
-        x[i][c] *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x[i][c]));  // silu
+        x[i][c] *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x[i][c]));
         if (ok[i]) ss += x[i][c] * x[i][c];
       }
-    }
+    return ss;
+  };
+  auto emit = [&](int t, float (&x)[NI][VEC], float ss) {
     if (grp) {
-      for (int o = a.lg >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
       const float f = (unit < a.nq ? a.qscale : 1.0f) / sqrtf(ss + a.eps);
       float* o = a.qk + ((int64_t)t * a.ng + unit) * a.dk - base;
 #pragma unroll
@@ -370,13 +302,124 @@ __global__ __launch_bounds__(256) void conv_silu_unit_kernel(ConvUnitArgs a) {
         }
       }
     }
+  };
+  float wk[TAPS > 0 ? TAPS : 1][NI][VEC], bs[NI][VEC];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+#pragma unroll
+    for (int c = 0; c < VEC; ++c) bs[i][c] = 0.f;
+    if (a.bias != nullptr) load_f(a.bias + ch[i], bs[i]);
+    if constexpr (TAPS > 0) {
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) load_f(a.w + (int64_t)k * a.C + ch[i], wk[k][i]);
+    }
+  }
+  int s = a.whole ? (int)blockIdx.x : a.seq_of[t_lo];
+  int s0 = a.cu[s], s1 = a.cu[s + 1], p0 = a.start[s];
+  if constexpr (TAPS > 0 && NI == 1 && WALK > 1) {
+    if (!a.whole && t_hi - t_lo == WALK && t_hi <= s1 && t_lo - s0 >= TAPS - 1) {
+      const T* up = u + (int64_t)(t_lo - (TAPS - 1)) * a.u_st + ch[0];
+      float r[WALK + TAPS - 1][VEC];
+#pragma unroll
+      for (int j = 0; j < WALK + TAPS - 1; ++j) {
+        load_row(up, r[j]);
+        up += a.u_st;
+      }
+      float x[WALK][1][VEC], ss[WALK];
+#pragma unroll
+      for (int j = 0; j < WALK; ++j) {
+#pragma unroll
+        for (int c = 0; c < VEC; ++c) {
+          float acc = bs[0][c];
+#pragma unroll
+          for (int k = 0; k < TAPS; ++k) acc += wk[k][0][c] * r[j + k][c];
+          x[j][0][c] = acc;
+        }
+        ss[j] = activate(x[j]);
+      }
+      if (grp) {
+#pragma unroll
+        for (int j = 0; j < WALK; ++j) ss[j] = unit_sum(ss[j], a.lg);
+      }
+#pragma unroll
+      for (int j = 0; j < WALK; ++j) emit(t_lo + j, x[j], ss[j]);
+      return;
+    }
+  }
+  // the input ``k`` positions before token t of the sequence that begins at row s0, position p0
+  auto past = [&](int t, int k, const float* st, int i, float* v) {
+    const int j = t - s0 - k;
+    if (j >= 0) {
+      load_row(u + (int64_t)(t - k) * a.u_st + ch[i], v);
+    } else if (p0 + j >= 0) {
+      load_f(st + (int64_t)(taps - 1 + j) * a.C + ch[i], v);
+    } else {
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) v[c] = 0.f;
+    }
+  };
+  float hist[NH][NI][VEC];  // hist[k]: the input k + 1 positions before the current token
+  float* st = a.state + (int64_t)a.sslot[s] * (taps - 1) * a.C;
+#pragma unroll 1
+  for (int t = t_lo; t < t_hi; ++t) {
+    bool reload = t == t_lo;
+    if (t >= s1) {
+      s = a.seq_of[t];
+      s0 = a.cu[s], s1 = a.cu[s + 1], p0 = a.start[s];
+      st = a.state + (int64_t)a.sslot[s] * (taps - 1) * a.C;
+      reload = true;
+    }
+    if constexpr (TAPS > 1) {
+      if (reload) {
+#pragma unroll
+        for (int k = 0; k < TAPS - 1; ++k)
+#pragma unroll
+          for (int i = 0; i < NI; ++i) past(t, k + 1, st, i, hist[k][i]);
+      }
+    }
+    float x[NI][VEC];
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      float cur[VEC];
+      load_row(u + (int64_t)t * a.u_st + ch[i], cur);
+      if constexpr (TAPS > 0) {  // (the oldest tap first, as on the other path)
+#pragma unroll
+        for (int c = 0; c < VEC; ++c) {
+          float acc = bs[i][c];
+#pragma unroll
+          for (int k = TAPS - 2; k >= 0; --k) acc += wk[TAPS - 2 - k][i][c] * hist[k][i][c];
+          x[i][c] = acc + wk[TAPS - 1][i][c] * cur[c];
+        }
+#pragma unroll
+        for (int k = TAPS - 2; k > 0; --k)
+#pragma unroll
+          for (int c = 0; c < VEC; ++c) hist[k][i][c] = hist[k - 1][i][c];
+        if constexpr (TAPS > 1) {
+#pragma unroll
+          for (int c = 0; c < VEC; ++c) hist[0][i][c] = cur[c];
+        }
+      } else {
+        float w1[VEC], v[VEC];
+        load_f(a.w + (int64_t)(taps - 1) * a.C + ch[i], w1);
+#pragma unroll
+        for (int c = 0; c < VEC; ++c) x[i][c] = bs[i][c] + w1[c] * cur[c];
+        for (int k = 1; k < taps; ++k) {
+          past(t, k, st, i, v);
+          load_f(a.w + (int64_t)(taps - 1 - k) * a.C + ch[i], w1);
+#pragma unroll
+          for (int c = 0; c < VEC; ++c) x[i][c] += w1[c] * v[c];
+        }
+      }
+    }
+    const float ss = activate(x);
+    emit(t, x, grp ? unit_sum(ss, a.lg) : 0.f);
   }
   if (a.whole) {  // the slot's new content; entry j is the input taps - 1 - j positions before the portion's end
     for (int j = 0; j < taps - 1; ++j) {
 #pragma unroll
       for (int i = 0; i < NI; ++i) {
         float v[VEC];
-        past(t_hi, taps - 1 - j, s0, p0, st, i, v);  // (ascending j reads entries that are not yet rewritten)
+        past(t_hi, taps - 1 - j, st, i, v);  // (ascending j reads entries that are not yet rewritten)
         if (ok[i]) {
 #pragma unroll
           for (int c = 0; c < VEC; ++c) st[(int64_t)j * a.C + ch[i] + c] = v[c];
@@ -424,25 +467,29 @@ std::tuple<at::Tensor, at::Tensor> conv_silu_unit(const at::Tensor& u, const at:
   const int NIv = ni > 1 ? 4 : 1;
   const int64_t span = (int64_t)lg * vec * NIv, units = ng + (C - ng * dk + span - 1) / span;
   const int64_t by = (units * lg + 255) / 256;
-  a.tok = 1;  // tokens per walk: as many as leave the chip a thousand workgroups
-  while (a.tok < CONV_WALK && T * by / (2 * a.tok) >= 1024) a.tok *= 2;
   HYB_CHECK(by <= 65535, "too many channels for one launch");
-  const dim3 grid((unsigned)(a.whole ? ns : (T + a.tok - 1) / a.tok), (unsigned)by);
+  // tokens per walk: 8 where that leaves the chip a thousand workgroups
+  const int walk = (T + 7) / 8 * by >= 1024 ? 8 : 4;
+  const dim3 grid((unsigned)(a.whole ? ns : (T + walk - 1) / walk), (unsigned)by);
   dispatch_act(u, [&](auto* tag) {
     using Tt = std::remove_pointer_t<decltype(tag)>;
     auto go = [&](auto kern) { kern<<<grid, 256, 0, cur_stream()>>>(a); };
-    auto taps_of = [&](auto vc, auto nc) {
-      constexpr int V = decltype(vc)::value, N = decltype(nc)::value;
+    auto taps_of = [&](auto vc, auto nc, auto wc) {
+      constexpr int V = decltype(vc)::value, N = decltype(nc)::value, WK = decltype(wc)::value;
       switch (taps) {
-        case 2: go(conv_silu_unit_kernel<Tt, V, N, 2>); break;
-        case 3: go(conv_silu_unit_kernel<Tt, V, N, 3>); break;
-        case 4: go(conv_silu_unit_kernel<Tt, V, N, 4>); break;
-        default: go(conv_silu_unit_kernel<Tt, V, N, 0>); break;
+        case 2: go(conv_silu_unit_kernel<Tt, V, N, 2, WK>); break;
+        case 3: go(conv_silu_unit_kernel<Tt, V, N, 3, WK>); break;
+        case 4: go(conv_silu_unit_kernel<Tt, V, N, 4, WK>); break;
+        default: go(conv_silu_unit_kernel<Tt, V, N, 0, WK>); break;
       }
     };
-    if (v4) taps_of(std::integral_constant<int, 4>(), std::integral_constant<int, 1>());
-    else if (NIv == 1) taps_of(std::integral_constant<int, 1>(), std::integral_constant<int, 1>());
-    else taps_of(std::integral_constant<int, 1>(), std::integral_constant<int, 4>());
+    auto sized = [&](auto vc, auto nc) {
+      if (walk == 8) taps_of(vc, nc, std::integral_constant<int, 8>());
+      else taps_of(vc, nc, std::integral_constant<int, 4>());
+    };
+    if (v4) sized(std::integral_constant<int, 4>(), std::integral_constant<int, 1>());
+    else if (NIv == 1) sized(std::integral_constant<int, 1>(), std::integral_constant<int, 1>());
+    else sized(std::integral_constant<int, 1>(), std::integral_constant<int, 4>());
     if (!a.whole && taps > 1)
       causal_conv_state_kernel<Tt><<<dim3((unsigned)ns, (unsigned)((C + 255) / 256)), 256, 0, cur_stream()>>>(
           (const Tt*)u.data_ptr(), u.stride(0), state.data_ptr<float>(), cu.data_ptr<int>(), start.data_ptr<int>(), sslot.data_ptr<int>(), (int)C, (int)taps);
