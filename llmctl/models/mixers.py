@@ -747,10 +747,11 @@ def _own_states(state):
 
 
 class GatedDeltaRule(nn.Module):
-    """The gated delta rule: per head a memory ``S [dim, vdim]`` with one decay per head and token, ``S <- g S``, ``u = beta (v -
-    S^T k)``, ``S <- S + k u^T``, ``o = S^T q``.  q, k (``kv_heads`` of them) and v pass short causal convolutions and silu;
-    q and k become unit vectors per head (``x / sqrt(sum x^2 + key_eps)``), q times ``dim^-1/2``; ``beta = sigmoid(W_b h)``, ``g =
-    exp(-exp(A_log) softplus(W_a h + dt_bias))``.  Each head's ``o`` over its root mean square, times one weight of vdim for
+    """The gated delta rule: per head a memory ``M_t = g_t M_(t-1) + k_t u_t^T`` of ``[dim, vdim]`` with ``u_t = beta_t (v_t - g_t M_(t-1)^T
+    k_t)``, read out as ``o_t = M_t^T q_t``: what the decayed memory already gives for a key is taken off before the write.  q, k
+    (``kv_heads`` of them) and v pass short causal convolutions and silu; the heads of q and k are brought to unit length
+    (squared length plus ``key_eps`` under the root), those of q times ``dim^-1/2``; ``beta = sigmoid(W_b h)``, ``log g = -exp(A_log)
+    softplus(W_a h + dt_bias)``.  Each head's ``o`` over its root mean square, times one weight of vdim for
     all heads, times ``silu(W_g h)``, then ``W_o``.  The fused input weight is ``[W_q ; W_k ; W_v ; W_g ; W_a ; W_b]``; state:
     the memory (fp32) and the convolutions' last inputs."""
 
@@ -796,10 +797,11 @@ class GatedDeltaRule(nn.Module):
 
 
 class Mamba2(nn.Module):
-    """Mamba-2 (state-space duality): ``W_in h = [z | x | B | C | dt]``; x, B and C pass a short causal convolution with bias and
-    silu; ``dt = softplus(dt + dt_bias)``; per head ``S [state, vdim]``: ``S_t = exp(-exp(A_log) dt) S_(t-1) + dt B x^T``, ``y = S^T C +
-    D x`` with B and C shared by the heads of one of ``groups`` groups.  The heads are concatenated, multiplied by ``silu(z)``
-    and then RMS-normed in ``norm_groups`` equal parts, times a weight; ``W_o``.  State: the memory (fp32) and the
+    """Mamba-2 (state-space duality): ``W_in h = [z | x | B | C | dt]``, where x, B and C pass one short causal convolution with
+    bias and silu.  Per head a memory ``M_t = e^(a_t) M_(t-1) + s_t B_t x_t^T`` of ``[state, vdim]`` with the step ``s = softplus(dt +
+    dt_bias)`` and ``a = -exp(A_log) s``, read out as ``M_t^T C_t + D x_t``; B and C are shared by the heads of one of ``groups``
+    groups.  All heads side by side times ``silu(z)`` go through an RMS norm of ``norm_groups`` equal parts with a weight, then
+    ``W_o``.  State: the memory (fp32) and the
     convolution's last inputs."""
 
     def __init__(self, width: int, heads: int, vdim: int, state: int, groups: int, taps: int, norm_groups: int, eps: float,
@@ -844,8 +846,8 @@ class Mamba2(nn.Module):
 
 
 class Retention(nn.Module):
-    """Retention: linear attention with a fixed decay per head and neither softmax nor denominator, ``S_t = decay_h S_(t-1) + k v^T``,
-    ``o = S^T q``; rotary on q and k (half pairs unless ``interleaved``), k times ``dim^-1/2`` after it.  Each head's ``o`` over its
+    """Retention: a memory ``M_t = decay_h M_(t-1) + k_t v_t^T`` per head with a constant factor, read out as ``M_t^T q_t``, without softmax
+    or denominator; rotary on q and k (half pairs unless ``interleaved``), then k times ``dim^-1/2``.  A head's read-out over its
     root mean square (no weight), times ``silu(W_g h)``, then ``W_o``.  The fused input weight is ``[W_q ; W_k ; W_v ; W_g]``; the
     memory is fp32 and lives in a state slot."""
 

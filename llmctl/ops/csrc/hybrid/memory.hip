@@ -1,5 +1,5 @@
 // Matrix memories with one decay per head and token: per (sequence, head) a memory S [dk, dv] (fp32) with
-//   S <- g S,   u = beta (v - S^T k) or beta v,   S <- S + k u^T,   o = S^T q (+ skip v),
+//   S_t = g_t S_(t-1) + k_t u_t^T,   u_t = beta_t v_t or beta_t (v_t - g_t S_(t-1)^T k_t),   o_t = S_t^T q_t (+ skip v_t),
 // the decay g and the write strength beta formed here in fp32 (kinds: 0 fixed decay and beta = 1; 1 state-space: beta = dt =
 // softplus(ga + dt_bias), g = exp(-exp(a_log) dt); 2 delta: g likewise, beta = sigmoid(gb), and the subtracting form of u).
 //

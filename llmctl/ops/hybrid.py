@@ -1,9 +1,10 @@
 """Ops of the hybrid sequence mixers: latent attention (compressed K/V cache, sliding window,
 softmax sink), grouped attention over paged rows (softmax or sigmoid weights, distance penalty), the
-mLSTM matrix memory, gated linear attention, the generalized delta rule, differential attention, the minGRU
-recurrence, the group-limited sigmoid router and the softmax router with a selection bias (optionally group-limited), and
-the fp32 residual stream of parallel layers, of layers with a gated residual between two norms, of layers over several
-residual streams (hyper-connections), and of layers whose sublayers read a causally convolved, group-normed input.
+mLSTM matrix memory, gated linear attention, the generalized delta rule, matrix memories with one decay per head and
+token (gated delta rule, state-space duality, retention), differential attention, the minGRU recurrence, the
+group-limited sigmoid router and the softmax router with a selection bias (optionally group-limited), and the fp32 residual stream of parallel layers, of layers with a gated residual between two norms, of layers over several
+residual streams (hyper-connections), of layers whose sublayers read a causally convolved, group-normed input, and of layers whose
+sublayers are normed on their way out only.
 
 GPU tensors run the HIP kernels of ``csrc/hybrid`` (``torch.ops.llmctl_hybrid.*``, library
 ``_llmctl_hybrid.so``); CPU tensors run :mod:`llmctl.ops.ref_hybrid`.  All activations are
@@ -605,8 +606,9 @@ def _memory_plan(b, device):
 
 
 def memory_scan(q, k, v, kind: str, S, b, ga=None, gb=None, a_log=None, dt_bias=None, log_decay=None, skip=None, norm=None):
-    """A matrix memory per head with one decay per head and token, over the step's tokens: ``S <- g S``, ``S <- S + k u^T``,
-    ``o = S^T q`` with ``u = beta v``, or ``u = beta (v - S^T k)`` (what the decayed memory gives for k is taken off first).
+    """A matrix memory per head with one decay per head and token, over the step's tokens: ``S_t = g_t S_(t-1) + k_t u_t^T``, ``o_t =
+    S_t^T q_t`` with ``u_t = beta_t v_t``, or ``u_t = beta_t (v_t - g_t S_(t-1)^T k_t)`` (what the decayed memory gives for k is
+    taken off first).
 
     ``kind`` says where g and beta come from (fp32 here): ``fixed``: ``g = exp(log_decay_h)``, beta = 1; ``ssm``: ``beta = dt =
     softplus(ga + dt_bias)``, ``g = exp(-exp(a_log) dt)``; ``delta``: g likewise, ``beta = sigmoid(gb)`` and the subtracting
@@ -659,7 +661,7 @@ def memory_scan(q, k, v, kind: str, S, b, ga=None, gb=None, a_log=None, dt_bias=
 
 def gate_groupnorm(o, z, w, groups: int, eps: float, out_dtype):
     """``y = o silu(z)`` (o fp32 ``[T, C]``, z ``[T, C]``), then an RMS norm of y in ``groups`` equal consecutive parts, each
-    over its own root mean square, the whole times ``w [C]``: the gate comes before the norm."""
+    over its own root mean square, the whole times ``w [C]``."""
     if use_native(o):
         return native_hybrid().gate_groupnorm(o, z, w, groups, eps, out_dtype == torch.bfloat16)
     return ref.gate_groupnorm(o, z, w, groups, eps, out_dtype)

@@ -507,8 +507,8 @@ def memory_gates(kind, T, H, ga, gb, a_log, dt_bias, log_decay):
 
 
 def memory_scan(q, k, v, kind, ga, gb, a_log, dt_bias, log_decay, skip, S, state_slots, cu, start):
-    """Token by token: S <- g S; u = beta (v - S^T k) (kind "delta") or beta v; S <- S + k u^T; o = S^T q (+ skip v).  The
-    state pool S [slots, H, dk, dv] (fp32) is read at ``state_slots[seq]`` (zeros when the sequence starts at position
+    """Token by token: the memory decays, takes ``k u^T`` in (u = beta v, less what the decayed memory gives for k in the kind
+    "delta") and is read out with q (+ skip v).  The state pool S [slots, H, dk, dv] (fp32) is read at ``state_slots[seq]`` (zeros when the sequence starts at position
     0) and written back after the sequence's last token of this step."""
     T, H, dv = v.shape
     rep = H // q.shape[1]

@@ -158,7 +158,7 @@ def test_mamba2_sizes(tmp_path, dev, sizes):
     check(tmp_path, dev, cfg, r, [[("a", 70), ("b", 2)], [("a", 1), ("b", 1)], [("a", 19), ("b", 1)]])
 
 
-def test_the_gate_comes_before_the_norm(tmp_path, dev):
+def test_gate_ahead_of_the_grouped_norm(tmp_path, dev):
     # gates that differ by orders of magnitude between the norm's groups and inside them
     cfg = U.config([(U.ssm(norm_groups=2), None)])
     W = U.random_weights(cfg, 12)
